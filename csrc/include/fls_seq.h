@@ -15,16 +15,21 @@ int fls_seq_version(void);
 // groups > 1 with offs == null: strided batch g: A + (g % a_mod) * a_gs, W + g * w_gs, C / bias + g * c_gs.
 // offs != null: row groups: group g owns rows [offs[g], offs[g+1]) of A and C and weight W + g * w_gs;
 // M is then the total row count (the bound of every group's rows).
-// Epilogue: + bias, then xIELU when act != null (act = {p, q}), stored as type tc (fp32, or bf16 when the
+// Epilogue: + bias, then an activation (act_kind 0: none; 1: xIELU, act = {p, q} on the device; 2: max(z, 0)^2), stored as type tc (fp32, or bf16 when the
 // consumer is the next product).
 int fls_seq_gemm(const void* A, int ta, const void* W, int tw, void* C, int tc, const float* bias, const float* act,
-                 int M, int N, int K, int lda, int ldw, int ldc, int groups, const int* offs, long long a_gs,
+                 int act_kind, int M, int N, int K, int lda, int ldw, int ldc, int groups, const int* offs, long long a_gs,
                  int a_mod, long long w_gs, long long c_gs, fls_stream_t s);
 // y[r] = w * x[row] / sqrt(mean_g(x[row]^2) + eps) per group of D / groups columns, row = idx ? idx[r] : r.
 // add != 0: y (fp32) += instead (the residual update), ty ignored.  woff is added to the weight (1 for
-// weights stored around zero).
+// weights stored around zero).  w_one != 0: w is one number for all columns.
 int fls_seq_group_rmsnorm(const float* x, int ldx, const int* idx, const float* w, void* y, int ty, int ldy,
-                          int rows, int D, int groups, float eps, int add, float woff, fls_stream_t s);
+                          int rows, int D, int groups, float eps, int add, float woff, int w_one, fls_stream_t s);
+// new = (keep ? x : 0) + coef (rms(a) wa + rms(b) wb) + f (all fp32 rows; a and b nullable together, f nullable), x <- new;
+// h != null: h = rms(new) hw as type th, hw a vector or (hw_one) one number
+int fls_seq_residual_branches(float* x, int ldx, int keep, const float* a, int lda, const float* wa, const float* b,
+                              int ldb, const float* wb, float coef, const float* f, int ldf, void* h, int th, int ldh,
+                              const float* hw, int hw_one, int rows, int D, float eps, fls_stream_t s);
 // out[t] = table[ids[t]] * scale (fp32 rows of the residual stream)
 int fls_seq_embed(const int* ids, const void* table, int tt, float* out, int T, int D, int V, float scale, fls_stream_t s);
 // Dynamic Tanh norm: y[r, c] = tanh(alpha[0] x[row, c]) wb[c] + wb[D + c], row = idx ? idx[r] : r; y of type ty
@@ -70,12 +75,16 @@ int fls_seq_kv_store(const float* k, int ldk, const float* kn, float eps, const 
 // the output of (row, head) times sigmoid(head_gate[t, h]).
 // out of type to (fp32 over bf16 pools allowed).  Gv (0: G), a divisor of G: the value pool holds Gv heads and key head g
 // reads value head g % Gv (several score maps over the same values).
+// pool_P > 0 (plain softmax over a window only): the softmax also runs over the mean key and value of every block of
+// pool_P positions that ends before the window (block b: positions b pool_P ..; seen by position i if (b + 1) pool_P - 1 <=
+// i - window), rows of the block pools kp / vp (ldkp / ldvp wide, page_size blocks a page, pages block_table[request])
 int fls_seq_attn_paged(const void* q, int ldq, int tq, const void* kc, int ldk, const void* vc, int ldv, int tc,
                        void* out, int to, int ldo, const int* tok_seq, const int* tok_pos, const int* page_table,
                        int pt_stride, int T, int H, int G, int d, int dv, float scale, float softcap,
                        const float* r1, const float* r2, int chunk, int window, int keep_first,
                        const float* gate_bias, float out_scale, int page_size, int nsplit, float* part,
-                       int has_sink, float sink, const float* head_gate, int ldhg, int Gv, fls_stream_t s);
+                       int has_sink, float sink, const float* head_gate, int ldhg, int Gv, int pool_P, const void* kp,
+                       int ldkp, const void* vp, int ldvp, const int* block_table, int bt_stride, fls_stream_t s);
 // the same attention on the matrix cores for bf16 pools and rows in tiles: tiles[n_tiles][2] = (first packed
 // row, rows <= 128) of one request each, covering every row of the step; q of type tq.  -2: shape not
 // served (use the above)
@@ -84,7 +93,8 @@ int fls_seq_attn_prefill(const void* q, int ldq, int tq, const void* kc, int ldk
                          const int* page_table, int pt_stride, int H, int G, int d, int dv, float scale,
                          float softcap, const float* r1, const float* r2, int chunk, int window, int keep_first,
                          const float* gate_bias, float out_scale, int page_size, int has_sink, float sink,
-                         const float* head_gate, int ldhg, int Gv, fls_stream_t s);
+                         const float* head_gate, int ldhg, int Gv, int pool_P, const void* kp, int ldkp, const void* vp,
+                         int ldvp, const int* block_table, int bt_stride, fls_stream_t s);
 // softmax attention of few rows whose H / G <= 32 query heads per key / value head become the columns of one
 // matrix-core tile (decode steps over cached latent rows): fp32 q, bf16 pools and out, window and kept first
 // keys as above; nsplit ranges of key tiles per row, part: T H nsplit (dv + 4) floats.  -2: shape not served
@@ -103,12 +113,21 @@ int fls_seq_causal_conv(const float* x, int ldx, const float* w, const float* b,
 // over their first rot entries (angle tok_pos * freqs[i]) and divided by sqrt(mean(head^2) + eps), q to qo (fp32
 // [T, H d]), k and v (v as convolved) to row kv_slot[t] of pools of type tc.  G = 0: queries only.  d, dv <= 512.
 // Gv (< 0: G): the row holds Gv value heads after its G key heads.  qnw / knw (nullable, [d]): the q / k heads are instead
-// RMS-normed BEFORE the rotation, times that weight (x / rms(x) * w, then rotated).
+// RMS-normed BEFORE the rotation, times that weight (x / rms(x) * w, then rotated).  no_norm != 0: only rotated.  half != 0: the
+// pairs are (i, i + rot / 2); amp: a factor on every cosine and sine.  P > 0 (every request brings one row): a row that
+// completes a block of P positions also writes the block's mean key and value (see fls_seq_block_means).
 int fls_seq_qkv_conv_rope(const float* z, int ldz, const float* w, float* state, int taps, const int* tok_seq,
                           const int* tok_pos, const int* cu, const int* pos0, const int* slot, const int* kv_slot,
                           int T, int B, int H, int G, int d, int dv, float eps, const float* freqs, int rot, float* qo,
                           int ldq, void* kc, int ldk, void* vc, int ldv, int tc, int one_row_each, int Gv, const float* qnw,
-                          const float* knw, fls_stream_t s);
+                          const float* knw, int half, float amp, int no_norm, const int* page_table, int pt_stride,
+                          int page_size, int P, void* kp, int ldkp, void* vp, int ldvp, const int* block_table, int bt_stride,
+                          fls_stream_t s);
+// the blocks of P positions that this step's rows complete: mean key and mean value of the P rows as pools kc / vc (type tc)
+// hold them (kcols / vcols columns, fp32 sums in position order), written to the block pools kp / vp (pages block_table)
+int fls_seq_block_means(const void* kc, int ldk, const void* vc, int ldv, int tc, const int* cu, const int* pos0, int B,
+                        int max_rows, int kcols, int vcols, const int* page_table, int pt_stride, int page_size, int P,
+                        void* kp, int ldkp, void* vp, int ldvp, const int* block_table, int bt_stride, fls_stream_t s);
 // generalized delta rule, per head a state S[d][d] in state[slot][H][d][d]:
 // S_t = diag(w) S_(t-1) - (a * u)(u^T S_(t-1)) + k v^T, o = S_t^T r; u = k / sqrt(sum k^2 + key_eps),
 // w = exp(-decay_scale sigmoid(wz + w0)), a = sigmoid(az); out = out_scale o / rms_head(o; norm_eps) norm_w sigmoid(g).

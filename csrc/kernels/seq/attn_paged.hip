@@ -5,7 +5,9 @@
 // G dv columns of pool rows ldk and ldv wide, so both may be one pool (values = a prefix of the keys:
 // attention over latent rows).  The query may be fp32 while the pools hold bf16.  has_sink: the softmax
 // has one more entry of score `sink` and no value (p_j = exp(s_j) / (exp(sink) + sum exp(s))); head_gate
-// [T, H] fp32: the output of (row, head) times sigmoid(head_gate[t, h]).
+// [T, H] fp32: the output of (row, head) times sigmoid(head_gate[t, h]).  Pooled blocks (pool_P > 0, beside a window):
+// the softmax also runs over one mean key and value for each block of pool_P positions that ends before the window,
+// read from block pools with pages of their own.
 //
 // One block (four wavefronts) per (row, query head).  The row's query sits in LDS as fp32.  The keys
 // it may see -- j <= i, inside its chunk of the sequence and / or its window -- are walked in tiles of
@@ -49,7 +51,7 @@ __device__ __forceinline__ float dot_row(const T* __restrict__ k, const float* _
   return acc;
 }
 
-template <typename TQ, typename T, typename TO>
+template <typename TQ, typename T, typename TO, bool POOL>
 __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ q, int ldq, const T* kc, int ldk,
                                                          const T* vc, int ldv, TO* __restrict__ out, int ldo,
                                                          const int* __restrict__ tok_seq, const int* __restrict__ tok_pos,
@@ -59,7 +61,8 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
                                                          int chunk, int window, int keep_first,
                                                          const float* __restrict__ gate_bias, float out_scale,
                                                          int page_size, int vec, float* __restrict__ part, int has_sink,
-                                                         float sink, const float* __restrict__ head_gate, int ldhg, int Gv) {
+                                                         float sink, const float* __restrict__ head_gate, int ldhg, int Gv,
+                                                         AttnBlocks ab) {
   __shared__ float qs[MAX_D];
   __shared__ float pw[4][64];
   __shared__ int prow[4][64];
@@ -75,7 +78,9 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
   __syncthreads();
   int lo = chunk > 0 ? (i / chunk) * chunk : 0;
   if (window > 0 && i - window + 1 > lo) lo = i - window + 1;
-  const int nkeep = min(keep_first, lo);          // kept first keys that the window no longer covers
+  // what precedes the window's keys: kept first keys that the window no longer covers, or the seen blocks
+  const int nkeep = POOL ? (i - window + 1 > 0 ? (i - window + 1) / ab.P : 0) : min(keep_first, lo);
+  const int* btable = POOL ? ab.table + (size_t)tok_seq[t] * ab.t_stride : nullptr;
   const int nkeys = nkeep + i - lo + 1;
   const int ntiles = (nkeys + 63) / 64;
   const float a1 = r1 != nullptr ? r1[h] : 0.f, a2 = r2 != nullptr ? r2[h] : 0.f;
@@ -97,8 +102,14 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
     float sc = -1e30f;
     int row = 0;
     if (valid) {
-      row = table[j / page_size] * page_size + j % page_size;
-      sc = dot_row<T>(kc + (size_t)row * ldk + (size_t)g * d, qs, d, vec) * scale;
+      if (POOL && n < nkeep) {
+        row = btable[n / page_size] * page_size + n % page_size;
+        sc = dot_row<T>(reinterpret_cast<const T*>(ab.kp) + (size_t)row * ab.ldk + (size_t)g * d, qs, d, vec) * scale;
+        row = ~row;                                // (a row of the block pools)
+      } else {
+        row = table[j / page_size] * page_size + j % page_size;
+        sc = dot_row<T>(kc + (size_t)row * ldk + (size_t)g * d, qs, d, vec) * scale;
+      }
       if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
       if (a1 != 0.f) sc -= a1 * log1pf(a2 * (float)(i - j));
     }
@@ -119,6 +130,10 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
     const int nk = min(64, nkeys - tile * 64);
+    auto vrow = [&](int r) -> const T* {
+      if (POOL && r < 0) return reinterpret_cast<const T*>(ab.vp) + (size_t)(~r) * ab.ldv + (size_t)gv * dv;
+      return vc + (size_t)r * ldv + (size_t)gv * dv;
+    };
 #pragma unroll
     for (int c = 0; c < MAX_DV_PER_LANE; ++c) {
       const int e = lane + 64 * c;
@@ -128,11 +143,11 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
         for (; jj + 8 <= nk; jj += 8) {            // eight independent value loads in flight
           float v[8];
 #pragma unroll
-          for (int x = 0; x < 8; ++x) v[x] = ldf(vc + (size_t)prow[wave][jj + x] * ldv + (size_t)gv * dv, e);
+          for (int x = 0; x < 8; ++x) v[x] = ldf(vrow(prow[wave][jj + x]), e);
 #pragma unroll
           for (int x = 0; x < 8; ++x) a += pw[wave][jj + x] * v[x];
         }
-        for (; jj < nk; ++jj) a += pw[wave][jj] * ldf(vc + (size_t)prow[wave][jj] * ldv + (size_t)gv * dv, e);
+        for (; jj < nk; ++jj) a += pw[wave][jj] * ldf(vrow(prow[wave][jj]), e);
         acc[c] = a;
       }
     }
@@ -225,7 +240,8 @@ extern "C" int fls_seq_attn_paged(const void* q, int ldq, int tq, const void* kc
                                   int pt_stride, int T, int H, int G, int d, int dv, float scale, float softcap,
                                   const float* r1, const float* r2, int chunk, int window, int keep_first,
                                   const float* gate_bias, float out_scale, int page_size, int nsplit, float* part,
-                                  int has_sink, float sink, const float* head_gate, int ldhg, int Gv, fls_stream_t s) {
+                                  int has_sink, float sink, const float* head_gate, int ldhg, int Gv, int pool_P, const void* kp,
+                                  int ldkp, const void* vp, int ldvp, const int* block_table, int bt_stride, fls_stream_t s) {
   if (T <= 0) return 0;
   if (Gv <= 0) Gv = G;
   if (G % Gv || (to == 1 && tc == 0)) return -1;
@@ -233,29 +249,39 @@ extern "C" int fls_seq_attn_paged(const void* q, int ldq, int tq, const void* kc
   if (nsplit < 1 || nsplit > MERGE_MAX_SPLIT || (nsplit > 1 && part == nullptr)) return -1;
   if (d > MAX_D || dv > 64 * MAX_DV_PER_LANE || G < 1 || H % G || page_size < 1 || G * d > ldk || Gv * dv > ldv || keep_first < 0
       || (tq == 1 && tc == 0)) return -1;
+  if (pool_P < 0 || (pool_P > 0 && (window < 1 || chunk > 0 || keep_first > 0 || has_sink || gate_bias != nullptr || r1 != nullptr ||
+                                    kp == nullptr || vp == nullptr || block_table == nullptr || G * d > ldkp || Gv * dv > ldvp)))
+    return -1;                                          // (blocks go with a plain softmax over a window)
+  const AttnBlocks ab = {pool_P, kp, ldkp, vp, ldvp, block_table, bt_stride};
   dim3 grid(H, T, nsplit);
   hipStream_t st = (hipStream_t)s;
 #define ATTN_PAGED_ARGS ldq, (const TC*)kc, ldk, (const TC*)vc, ldv, (TOUT*)out, ldo, tok_seq, tok_pos, page_table, pt_stride, H, G, \
                         d, dv, scale, softcap, r1, r2, chunk, window, keep_first, gate_bias, out_scale, page_size, vec, part, has_sink, sink, \
-                        nsplit > 1 ? nullptr : head_gate, ldhg, Gv
+                        nsplit > 1 ? nullptr : head_gate, ldhg, Gv, ab
+#define ATTN_PAGED_GO(TQ)                                                                                                   \
+  do {                                                                                                                      \
+    if (pool_P > 0) hipLaunchKernelGGL((attn_paged_kernel<TQ, TC, TOUT, true>), grid, dim3(256), 0, st, (const TQ*)q, ATTN_PAGED_ARGS); \
+    else hipLaunchKernelGGL((attn_paged_kernel<TQ, TC, TOUT, false>), grid, dim3(256), 0, st, (const TQ*)q, ATTN_PAGED_ARGS);           \
+  } while (0)
   if (tc == 1) {
     using TC = bf16_t;
-    const int vec = d % 8 == 0 && (uintptr_t)kc % 16 == 0 && ldk % 8 == 0;
+    const int vec = d % 8 == 0 && (uintptr_t)kc % 16 == 0 && ldk % 8 == 0 && (pool_P == 0 || ((uintptr_t)kp % 16 == 0 && ldkp % 8 == 0));
     if (to == 0) {
       using TOUT = float;
-      if (tq == 1) hipLaunchKernelGGL((attn_paged_kernel<bf16_t, bf16_t, float>), grid, dim3(256), 0, st, (const bf16_t*)q, ATTN_PAGED_ARGS);
-      else hipLaunchKernelGGL((attn_paged_kernel<float, bf16_t, float>), grid, dim3(256), 0, st, (const float*)q, ATTN_PAGED_ARGS);
+      if (tq == 1) ATTN_PAGED_GO(bf16_t);
+      else ATTN_PAGED_GO(float);
     } else {
       using TOUT = bf16_t;
-      if (tq == 1) hipLaunchKernelGGL((attn_paged_kernel<bf16_t, bf16_t, bf16_t>), grid, dim3(256), 0, st, (const bf16_t*)q, ATTN_PAGED_ARGS);
-      else hipLaunchKernelGGL((attn_paged_kernel<float, bf16_t, bf16_t>), grid, dim3(256), 0, st, (const float*)q, ATTN_PAGED_ARGS);
+      if (tq == 1) ATTN_PAGED_GO(bf16_t);
+      else ATTN_PAGED_GO(float);
     }
   } else {
     using TC = float;
     using TOUT = float;
-    const int vec = d % 4 == 0 && (uintptr_t)kc % 16 == 0 && ldk % 4 == 0;
-    hipLaunchKernelGGL((attn_paged_kernel<float, float, float>), grid, dim3(256), 0, st, (const float*)q, ATTN_PAGED_ARGS);
+    const int vec = d % 4 == 0 && (uintptr_t)kc % 16 == 0 && ldk % 4 == 0 && (pool_P == 0 || ((uintptr_t)kp % 16 == 0 && ldkp % 4 == 0));
+    ATTN_PAGED_GO(float);
   }
+#undef ATTN_PAGED_GO
 #undef ATTN_PAGED_ARGS
   SEQ_LAUNCH_CHECK();
   if (nsplit > 1) return seq_attn_merge(part, out, to, ldo, T, H, dv, nsplit, gate_bias != nullptr, out_scale, has_sink, sink, head_gate, ldhg, s);

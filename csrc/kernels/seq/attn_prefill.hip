@@ -4,6 +4,10 @@
 // bf16 on their way into the fragments).  Keys of a row tile: first the kept first keys that lie before
 // the tile's window (if any), then the window's keys, both walked 32 at a time.
 //
+// POOL (beside a window): ahead of the window's tiles come tiles of block means, one key and value for each block of
+// ab.P positions that ends before the window, from block pools with pages of their own; query i sees blocks
+// b < (i - window + 1) / ab.P.
+//
 // The host cuts every request's rows of the step into tiles of up to 128 consecutive rows; a block
 // serves one tile and one query head, its four waves 32 query rows each.  Keys are walked 32 at a
 // time, from the first key the tile's first row may see to the tile's last row, gathered from the
@@ -27,7 +31,7 @@ typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 #define KT 32             // keys per tile
 #define PLD (KT + 8)      // row stride (elements) of the transposed V tile and of the weight tiles
 
-template <int D, int DV, typename TQ, typename TO>
+template <int D, int DV, typename TQ, typename TO, bool POOL>
 __global__ __launch_bounds__(256) void attn_prefill_kernel(const TQ* __restrict__ q, int ldq, const bf16_t* __restrict__ kc, int ldk,
                                                            const bf16_t* __restrict__ vc, int ldv, TO* __restrict__ out, int ldo,
                                                            const int* __restrict__ tiles, const int* __restrict__ tok_seq,
@@ -37,7 +41,7 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const TQ* __restrict_
                                                            int chunk, int window, int keep_first,
                                                            const float* __restrict__ gate_bias, float out_scale, int page_size,
                                                            int has_sink, float sink, const float* __restrict__ head_gate,
-                                                           int ldhg, int Gv) {
+                                                           int ldhg, int Gv, AttnBlocks ab) {
   constexpr int KLD = D + 8;
   __shared__ __attribute__((aligned(16))) bf16_t Ks[KT * KLD];
   __shared__ __attribute__((aligned(16))) bf16_t Vt[DV * PLD];
@@ -92,26 +96,36 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const TQ* __restrict_
   const float inv_cap = softcap > 0.f ? 1.f / softcap : 0.f;
   // key tiles: nt_keep tiles over the kept first keys [0, nkeep) that lie before the block's window,
   // then the tiles from lo_blk to the block's last row
-  const int nkeep = min(keep_first, lo_blk);
+  // (POOL: instead nt_keep tiles over the blocks [0, nkeep) that the block's last row sees)
+  auto seen_blocks = [&](int i) { return i - window + 1 > 0 ? (i - window + 1) / ab.P : 0; };
+  const int nkeep = POOL ? seen_blocks(i_last) : min(keep_first, lo_blk);
+  const int keep_q = POOL ? seen_blocks(iq) : keep_first;            // what of them this lane's query sees ...
+  const int keep_w = POOL ? seen_blocks(w_last) : keep_first;        // ... and any of the wave's
+  const int* btable = POOL ? ab.table + (size_t)tok_seq[row0] * ab.t_stride : nullptr;
   const int nt_keep = (nkeep + KT - 1) / KT;
   const int nt = nt_keep + (i_last - lo_blk) / KT + 1;
   // K / V of a key tile travel global -> registers -> LDS; the next tile's loads are issued before this
   // tile's matrix work and land in LDS after it, so the page gather's latency hides under the MFMAs
-  constexpr int NK = KT * (D / 8) / 256, NV = KT * (DV / 8) / 256;
-  static_assert(NK >= 1 && NV >= 1, "a tile has at least one 16-byte piece per thread");
+  constexpr int PK = KT * (D / 8), PV = KT * (DV / 8);               // 16-byte pieces of a tile
+  constexpr int NK = (PK + 255) / 256, NV = (PV + 255) / 256;        // per thread (the last one of some threads may be none)
   uint4 kreg[NK], vreg[NV];
   auto fetch = [&](int ti) {
-    const int j0 = ti < nt_keep ? ti * KT : lo_blk + (ti - nt_keep) * KT;
-    const int jend = ti < nt_keep ? nkeep : i_last + 1;
+    const bool pre = ti < nt_keep;
+    const int j0 = pre ? ti * KT : lo_blk + (ti - nt_keep) * KT;
+    const int jend = pre ? nkeep : i_last + 1;
+    const int* tab = POOL && pre ? btable : table;
+    const bf16_t* kb = POOL && pre ? reinterpret_cast<const bf16_t*>(ab.kp) : kc;
+    const bf16_t* vb = POOL && pre ? reinterpret_cast<const bf16_t*>(ab.vp) : vc;
+    const int lk = POOL && pre ? ab.ldk : ldk, lv = POOL && pre ? ab.ldv : ldv;
 #pragma unroll
     for (int x = 0; x < NK; ++x) {
       const int e = threadIdx.x + 256 * x;
       const int kk = e / (D / 8), seg = e % (D / 8);
       const int j = j0 + kk;
       kreg[x] = make_uint4(0, 0, 0, 0);
-      if (j < jend) {
-        const size_t row = (size_t)table[j / page_size] * page_size + j % page_size;
-        kreg[x] = *reinterpret_cast<const uint4*>(kc + row * ldk + (size_t)g * D + seg * 8);
+      if (j < jend && (PK % 256 == 0 || e < PK)) {
+        const size_t row = (size_t)tab[j / page_size] * page_size + j % page_size;
+        kreg[x] = *reinterpret_cast<const uint4*>(kb + row * lk + (size_t)g * D + seg * 8);
       }
     }
 #pragma unroll
@@ -120,9 +134,9 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const TQ* __restrict_
       const int kk = e % KT, seg = e / KT;
       const int j = j0 + kk;
       vreg[x] = make_uint4(0, 0, 0, 0);
-      if (j < jend) {
-        const size_t row = (size_t)table[j / page_size] * page_size + j % page_size;
-        vreg[x] = *reinterpret_cast<const uint4*>(vc + row * ldv + (size_t)(g % Gv) * DV + seg * 8);
+      if (j < jend && (PV % 256 == 0 || e < PV)) {
+        const size_t row = (size_t)tab[j / page_size] * page_size + j % page_size;
+        vreg[x] = *reinterpret_cast<const uint4*>(vb + row * lv + (size_t)(g % Gv) * DV + seg * 8);
       }
     }
   };
@@ -135,19 +149,21 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const TQ* __restrict_
 #pragma unroll
     for (int x = 0; x < NK; ++x) {
       const int e = threadIdx.x + 256 * x;
-      *reinterpret_cast<uint4*>(Ks + (e / (D / 8)) * KLD + (e % (D / 8)) * 8) = kreg[x];
+      if (PK % 256 == 0 || e < PK) *reinterpret_cast<uint4*>(Ks + (e / (D / 8)) * KLD + (e % (D / 8)) * 8) = kreg[x];
     }
 #pragma unroll
     for (int x = 0; x < NV; ++x) {
       const int e = threadIdx.x + 256 * x;
       const int kk = e % KT, seg = e / KT;
       const bf16_t* ev = reinterpret_cast<const bf16_t*>(&vreg[x]);
+      if (PV % 256 != 0 && e >= PV) continue;
 #pragma unroll
       for (int y = 0; y < 8; ++y) Vt[(seg * 8 + y) * PLD + kk] = ev[y];
     }
     __syncthreads();
     if (ti + 1 < nt) fetch(ti + 1);
-    if (wave * 32 >= nrows || (!kept && (j0 > w_last || (j0 + KT - 1 < lo_w && j0 >= keep_first)))) continue;   // (wave-uniform)
+    if (wave * 32 >= nrows || (POOL && kept && j0 >= keep_w) ||
+        (!kept && (j0 > w_last || (j0 + KT - 1 < lo_w && (POOL || j0 >= keep_first))))) continue;   // (wave-uniform)
     floatx16 S;
 #pragma unroll
     for (int r = 0; r < 16; ++r) S[r] = 0.f;
@@ -165,7 +181,8 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const TQ* __restrict_
       float sc = S[r] * scale;
       if (softcap > 0.f) sc = softcap * (1.f - 2.f / (__expf(2.f * sc * inv_cap) + 1.f));
       if (a1 != 0.f) sc -= a1 * __logf(1.f + a2 * (float)max(iq - j, 0));
-      const bool vis = qok && j < jend && j <= iq && (j >= lo_q || j < keep_first);
+      const bool vis = POOL ? qok && (kept ? j < keep_q : j >= lo_q && j <= iq)
+                            : qok && j < jend && j <= iq && (j >= lo_q || j < keep_first);
       if (gated) p[r] = vis ? 1.f / (1.f + __expf(-(sc + gb))) : 0.f;
       else p[r] = vis ? sc : -1e30f;
       mt = fmaxf(mt, p[r]);
@@ -244,32 +261,52 @@ extern "C" int fls_seq_attn_prefill(const void* q, int ldq, int tq, const void* 
                                     const int* page_table, int pt_stride, int H, int G, int d, int dv, float scale,
                                     float softcap, const float* r1, const float* r2, int chunk, int window, int keep_first,
                                     const float* gate_bias, float out_scale, int page_size, int has_sink, float sink,
-                                    const float* head_gate, int ldhg, int Gv, fls_stream_t s) {
+                                    const float* head_gate, int ldhg, int Gv, int pool_P, const void* kp, int ldkp, const void* vp,
+                                    int ldvp, const int* block_table, int bt_stride, fls_stream_t s) {
   if (n_tiles <= 0) return 0;
   if (has_sink && gate_bias != nullptr) return -1;
   if (Gv <= 0) Gv = G;
   if (G < 1 || H % G || G % Gv || page_size < 1 || ldq % 8 || ldo % 4 || ldk % 8 || ldv % 8 || G * d > ldk || Gv * dv > ldv ||
       (uintptr_t)q % 16 || (uintptr_t)kc % 16 || (uintptr_t)vc % 16 || (uintptr_t)out % 16 || keep_first < 0)
     return -2;
+  if (pool_P < 0 || (pool_P > 0 && (window < 1 || chunk > 0 || keep_first > 0 || has_sink || gate_bias != nullptr || r1 != nullptr ||
+                                    kp == nullptr || vp == nullptr || block_table == nullptr || G * d > ldkp || Gv * dv > ldvp)))
+    return -1;                                          // (blocks go with a plain softmax over a window)
+  if (pool_P > 0 && (tq != 0 || ldkp % 8 || ldvp % 8 || (uintptr_t)kp % 16 || (uintptr_t)vp % 16)) return -2;
+  const AttnBlocks ab = {pool_P, kp, ldkp, vp, ldvp, block_table, bt_stride};
   dim3 grid(H, n_tiles);
   hipStream_t st = (hipStream_t)s;
-#define ATTN_PF_(DD, DDV, TQ_, TO_)                                                                                       \
-  hipLaunchKernelGGL((attn_prefill_kernel<DD, DDV, TQ_, TO_>), grid, dim3(256), 0, st, (const TQ_*)q, ldq,                \
+#define ATTN_PF_(DD, DDV, TQ_, TO_, PP)                                                                                   \
+  hipLaunchKernelGGL((attn_prefill_kernel<DD, DDV, TQ_, TO_, PP>), grid, dim3(256), 0, st, (const TQ_*)q, ldq,            \
                      (const bf16_t*)kc, ldk, (const bf16_t*)vc, ldv, (TO_*)out, ldo, tiles, tok_seq, tok_pos,             \
                      page_table, pt_stride, H, G, scale, softcap, r1, r2, chunk, window, keep_first, gate_bias,           \
-                     out_scale, page_size, has_sink, sink, head_gate, ldhg, Gv)
+                     out_scale, page_size, has_sink, sink, head_gate, ldhg, Gv, ab)
 #define ATTN_PF(DD, DDV)                                                                                                  \
   do {                                                                                                                    \
-    if (tq == 1 && to == 1) ATTN_PF_(DD, DDV, bf16_t, bf16_t);                                                            \
-    else if (tq == 1) ATTN_PF_(DD, DDV, bf16_t, float);                                                                   \
-    else if (to == 1) ATTN_PF_(DD, DDV, float, bf16_t);                                                                   \
-    else ATTN_PF_(DD, DDV, float, float);                                                                                 \
+    if (tq == 1 && to == 1) ATTN_PF_(DD, DDV, bf16_t, bf16_t, false);                                                     \
+    else if (tq == 1) ATTN_PF_(DD, DDV, bf16_t, float, false);                                                            \
+    else if (to == 1) ATTN_PF_(DD, DDV, float, bf16_t, false);                                                            \
+    else ATTN_PF_(DD, DDV, float, float, false);                                                                          \
   } while (0)
-  if (d == 128 && dv == 128) ATTN_PF(128, 128);
+#define ATTN_PF_POOL(DD, DDV)                                                                                             \
+  do {                                                                                                                    \
+    if (to == 1) ATTN_PF_(DD, DDV, float, bf16_t, true);                                                                  \
+    else ATTN_PF_(DD, DDV, float, float, true);                                                                           \
+  } while (0)
+  if (pool_P > 0) {
+    if (d == 128 && dv == 128) ATTN_PF_POOL(128, 128);
+    else if (d == 96 && dv == 96) ATTN_PF_POOL(96, 96);
+    else if (d == 64 && dv == 64) ATTN_PF_POOL(64, 64);
+    else if (d == 32 && dv == 32) ATTN_PF_POOL(32, 32);
+    else if (d == 128 && dv == 64) ATTN_PF_POOL(128, 64);
+    else if (d == 64 && dv == 128) ATTN_PF_POOL(64, 128);
+    else return -2;
+  } else if (d == 128 && dv == 128) ATTN_PF(128, 128);
   else if (d == 64 && dv == 64) ATTN_PF(64, 64);
   else if (d == 128 && dv == 64) ATTN_PF(128, 64);
   else if (d == 64 && dv == 128) ATTN_PF(64, 128);
   else return -2;
+#undef ATTN_PF_POOL
 #undef ATTN_PF
 #undef ATTN_PF_
   SEQ_LAUNCH_CHECK();

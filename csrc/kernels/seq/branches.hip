@@ -1,0 +1,160 @@
+// The residual row update of layers whose sublayers run side by side: two branches that join through norms of their
+// own, a plain addend, and the norm the next reader wants, in one pass over the row.
+//   new = (keep ? x : 0) + coef (rms(a) wa + rms(b) wb) + f;   x <- new;   h = rms(new) hw
+// (a, b, f and h each optional; hw is a vector, or one number for all columns).  All sums fp32.
+#include "seq_common.h"
+#include "fls_seq.h"
+
+#define RB_PIECES 8                // 256 VE columns a piece; that many pieces of a and b stay in registers
+
+template <int VE> struct RbVec { float v[VE]; };
+template <int VE>
+__device__ __forceinline__ RbVec<VE> rb_load(const float* p) {
+  RbVec<VE> r;
+  if constexpr (VE == 4) {
+    const float4 q = *reinterpret_cast<const float4*>(p);
+    r.v[0] = q.x; r.v[1] = q.y; r.v[2] = q.z; r.v[3] = q.w;
+  } else {
+    r.v[0] = p[0];
+  }
+  return r;
+}
+template <int VE>
+__device__ __forceinline__ void rb_store(float* p, const RbVec<VE>& r) {
+  if constexpr (VE == 4) *reinterpret_cast<float4*>(p) = make_float4(r.v[0], r.v[1], r.v[2], r.v[3]);
+  else p[0] = r.v[0];
+}
+template <int VE>
+__device__ __forceinline__ void rb_store(bf16_t* p, const RbVec<VE>& r) {
+  if constexpr (VE == 4) {
+    const bf16_t e[4] = {f_to_bf16(r.v[0]), f_to_bf16(r.v[1]), f_to_bf16(r.v[2]), f_to_bf16(r.v[3])};
+    *reinterpret_cast<uint2*>(p) = *reinterpret_cast<const uint2*>(e);
+  } else {
+    p[0] = f_to_bf16(r.v[0]);
+  }
+}
+
+// one block per row
+template <typename TO, int VE>
+__global__ __launch_bounds__(256) void residual_branches_kernel(float* __restrict__ x, int ldx, int keep, const float* __restrict__ a,
+                                                                int lda, const float* __restrict__ wa, const float* __restrict__ b,
+                                                                int ldb, const float* __restrict__ wb, float coef,
+                                                                const float* __restrict__ f, int ldf_, TO* __restrict__ h, int ldh,
+                                                                const float* __restrict__ hw, int hw_one, int D, float eps) {
+  __shared__ float red[8];
+  const int r = blockIdx.x;
+  const int wave = threadIdx.x >> 6;
+  float* xr = x + (size_t)r * ldx;
+  const float* ar = a != nullptr ? a + (size_t)r * lda : nullptr;
+  const float* br = a != nullptr ? b + (size_t)r * ldb : nullptr;
+  const float* fr = f != nullptr ? f + (size_t)r * ldf_ : nullptr;
+  const int np = (D + 256 * VE - 1) / (256 * VE);
+  RbVec<VE> av[RB_PIECES], bv[RB_PIECES];
+  float rsa = 0.f, rsb = 0.f;
+  if (ar != nullptr) {
+    float sa = 0.f, sb = 0.f;
+#pragma unroll
+    for (int k = 0; k < RB_PIECES; ++k) {
+      const int c = (threadIdx.x + 256 * k) * VE;
+      if (c < D) {
+        av[k] = rb_load<VE>(ar + c);
+        bv[k] = rb_load<VE>(br + c);
+#pragma unroll
+        for (int i = 0; i < VE; ++i) { sa += av[k].v[i] * av[k].v[i]; sb += bv[k].v[i] * bv[k].v[i]; }
+      }
+    }
+    for (int k = RB_PIECES; k < np; ++k) {
+      const int c = (threadIdx.x + 256 * k) * VE;
+      if (c < D) {
+        const RbVec<VE> ta = rb_load<VE>(ar + c), tb = rb_load<VE>(br + c);
+#pragma unroll
+        for (int i = 0; i < VE; ++i) { sa += ta.v[i] * ta.v[i]; sb += tb.v[i] * tb.v[i]; }
+      }
+    }
+    sa = wave_sum(sa);
+    sb = wave_sum(sb);
+    if ((threadIdx.x & 63) == 0) { red[wave] = sa; red[4 + wave] = sb; }
+    __syncthreads();
+    rsa = coef / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)D + eps);
+    rsb = coef / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)D + eps);
+    __syncthreads();
+  }
+  float ss = 0.f;
+  // one piece of the row; returns the new entries
+  auto piece = [&](int c, const RbVec<VE>& pa, const RbVec<VE>& pb) -> RbVec<VE> {
+    RbVec<VE> n;
+    if (keep) n = rb_load<VE>(xr + c);
+    else {
+#pragma unroll
+      for (int i = 0; i < VE; ++i) n.v[i] = 0.f;
+    }
+    if (ar != nullptr) {
+      const RbVec<VE> qa = rb_load<VE>(wa + c), qb = rb_load<VE>(wb + c);
+#pragma unroll
+      for (int i = 0; i < VE; ++i) n.v[i] += pa.v[i] * rsa * qa.v[i] + pb.v[i] * rsb * qb.v[i];
+    }
+    if (fr != nullptr) {
+      const RbVec<VE> q = rb_load<VE>(fr + c);
+#pragma unroll
+      for (int i = 0; i < VE; ++i) n.v[i] += q.v[i];
+    }
+    rb_store<VE>(xr + c, n);
+#pragma unroll
+    for (int i = 0; i < VE; ++i) ss += n.v[i] * n.v[i];
+    return n;
+  };
+#pragma unroll
+  for (int k = 0; k < RB_PIECES; ++k) {
+    const int c = (threadIdx.x + 256 * k) * VE;
+    if (c < D) av[k] = piece(c, av[k], bv[k]);       // (from here on av holds the new entries)
+  }
+  for (int k = RB_PIECES; k < np; ++k) {
+    const int c = (threadIdx.x + 256 * k) * VE;
+    if (c >= D) break;
+    RbVec<VE> ta, tb;
+    if (ar != nullptr) { ta = rb_load<VE>(ar + c); tb = rb_load<VE>(br + c); }
+    piece(c, ta, tb);
+  }
+  if (h == nullptr) return;
+  ss = wave_sum(ss);
+  if ((threadIdx.x & 63) == 0) red[wave] = ss;
+  __syncthreads();
+  const float rs = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)D + eps);
+  TO* hr = h + (size_t)r * ldh;
+  const float g1 = hw_one ? hw[0] : 0.f;
+  auto out = [&](int c, RbVec<VE> n) {
+#pragma unroll
+    for (int i = 0; i < VE; ++i) n.v[i] *= rs * (hw_one ? g1 : hw[c + i]);
+    rb_store<VE>(hr + c, n);
+  };
+#pragma unroll
+  for (int k = 0; k < RB_PIECES; ++k) {
+    const int c = (threadIdx.x + 256 * k) * VE;
+    if (c < D) out(c, av[k]);
+  }
+  for (int k = RB_PIECES; k < np; ++k) {             // (a thread re-reads only what it wrote itself)
+    const int c = (threadIdx.x + 256 * k) * VE;
+    if (c >= D) break;
+    out(c, rb_load<VE>(xr + c));
+  }
+}
+
+extern "C" int fls_seq_residual_branches(float* x, int ldx, int keep, const float* a, int lda, const float* wa, const float* b,
+                                         int ldb, const float* wb, float coef, const float* f, int ldf, void* h, int th, int ldh,
+                                         const float* hw, int hw_one, int rows, int D, float eps, fls_stream_t s) {
+  if (rows <= 0) return 0;
+  if (D < 1 || x == nullptr || (a == nullptr) != (b == nullptr) || (a != nullptr && (wa == nullptr || wb == nullptr)) ||
+      (h != nullptr && hw == nullptr))
+    return -1;
+  auto al = [](const void* p, int ld, int es) { return p == nullptr || ((uintptr_t)p % (4 * es) == 0 && ld % 4 == 0); };
+  const int vec = D % 4 == 0 && al(x, ldx, 4) && al(a, lda, 4) && al(b, ldb, 4) && al(wa, 0, 4) && al(wb, 0, 4) && al(f, ldf, 4) &&
+                  al(h, ldh, th == 1 ? 2 : 4);
+  hipStream_t st = (hipStream_t)s;
+#define RB_GO(TO, VV) hipLaunchKernelGGL((residual_branches_kernel<TO, VV>), dim3(rows), dim3(256), 0, st, x, ldx, keep, a, lda, wa, b, ldb, \
+                                         wb, coef, f, ldf, (TO*)h, ldh, hw, hw_one, D, eps)
+  if (th == 1) { if (vec) RB_GO(bf16_t, 4); else RB_GO(bf16_t, 1); }
+  else { if (vec) RB_GO(float, 4); else RB_GO(float, 1); }
+#undef RB_GO
+  SEQ_LAUNCH_CHECK();
+  return 0;
+}

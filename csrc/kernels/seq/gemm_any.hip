@@ -30,23 +30,25 @@ __device__ __forceinline__ void cvt_store(bf16_t* d, float v) { *d = f_to_bf16(v
 __device__ __forceinline__ void cvt_store(float* d, float v) { *d = v; }
 __device__ __forceinline__ void cvt_store(bf16_t* d, bf16_t v) { *d = v; }
 
-// What a kernel does with a finished accumulator element: + bias, optionally the xIELU activation
-// (act = {p, q}: z > 0: softplus(p) z^2 + z/2, else (1/2 + softplus(q)) (exp(z) - 1 - z) + z/2), then the
-// store as fp32 or bf16 -- so a projection whose consumer is the next matrix product writes that
+// What a kernel does with a finished accumulator element: + bias, optionally an activation (kind 1, xIELU with
+// act = {p, q}: z > 0: softplus(p) z^2 + z/2, else (1/2 + softplus(q)) (exp(z) - 1 - z) + z/2; kind 2: the square
+// of max(z, 0)), then the store as fp32 or bf16 -- so a projection whose consumer is the next matrix product writes that
 // product's operand directly and the fp32 intermediate never reaches memory.
 struct Epi {
   const float* bias;
-  const float* act;      // null: no activation
+  const float* act;      // the activation's numbers on the device, if it has any
+  int kind;              // 0 none, 1 xIELU, 2 squared ReLU
   int tc;                // element type of C: 0 fp32, 1 bf16
 };
 struct EpiRegs { float ap, an; };
 __device__ __forceinline__ EpiRegs epi_regs(const Epi& e) {
   EpiRegs r = {0.f, 0.f};
-  if (e.act != nullptr) { r.ap = softplus_f(e.act[0]); r.an = 0.5f + softplus_f(e.act[1]); }
+  if (e.kind == 1) { r.ap = softplus_f(e.act[0]); r.an = 0.5f + softplus_f(e.act[1]); }
   return r;
 }
 __device__ __forceinline__ void emit(void* C, size_t idx, float v, const Epi& e, const EpiRegs& r) {
-  if (e.act != nullptr) v = v > 0.f ? r.ap * v * v + 0.5f * v : r.an * (expm1f(v) - v) + 0.5f * v;
+  if (e.kind == 2) { v = fmaxf(v, 0.f); v *= v; }
+  else if (e.kind == 1) v = v > 0.f ? r.ap * v * v + 0.5f * v : r.an * (expm1f(v) - v) + 0.5f * v;
   if (e.tc == 1) reinterpret_cast<bf16_t*>(C)[idx] = f_to_bf16(v);
   else reinterpret_cast<float*>(C)[idx] = v;
 }
@@ -391,9 +393,10 @@ static void launch(int big, dim3 grid, hipStream_t st, const void* A, const void
 }
 
 extern "C" int fls_seq_gemm(const void* A, int ta, const void* W, int tw, void* C, int tc, const float* bias_p,
-                            const float* act, int M, int N, int K, int lda, int ldw, int ldc, int groups, const int* offs,
+                            const float* act, int act_kind, int M, int N, int K, int lda, int ldw, int ldc, int groups, const int* offs,
                             long long a_gs, int a_mod, long long w_gs, long long c_gs, fls_stream_t s) {
-  const Epi bias = {bias_p, act, tc};
+  if (act_kind < 0 || act_kind > 2 || (act_kind == 1 && act == nullptr)) return -1;
+  const Epi bias = {bias_p, act, act_kind, tc};
   if (M <= 0 || N <= 0) return 0;
   if (K <= 0 || groups < 1 || (ta == 1 && tw == 0)) return -1;
   const int ea = ta == 1 ? 2 : 4, ew = tw == 1 ? 2 : 4;

@@ -9,7 +9,7 @@
 template <typename TO, int ADD>
 __global__ __launch_bounds__(256) void group_rmsnorm_kernel(const float* __restrict__ x, int ldx, const int* __restrict__ idx,
                                                             const float* __restrict__ w, TO* __restrict__ y, int ldy,
-                                                            int D, int groups, float eps, float woff) {
+                                                            int D, int groups, float eps, float woff, int w_one) {
   __shared__ float red[4];
   const int r = blockIdx.x, g = blockIdx.y;
   const int n = D / groups;
@@ -21,20 +21,20 @@ __global__ __launch_bounds__(256) void group_rmsnorm_kernel(const float* __restr
   const float* wg = w + (size_t)g * n;
   TO* yr = y + (size_t)r * ldy + (size_t)g * n;
   for (int c = threadIdx.x; c < n; c += 256) {
-    const float v = xr[c] * rs * (wg[c] + woff);
+    const float v = xr[c] * rs * ((w_one ? w[0] : wg[c]) + woff);
     if constexpr (ADD) yr[c] += v; else stf(yr, c, v);
   }
 }
 
 extern "C" int fls_seq_group_rmsnorm(const float* x, int ldx, const int* idx, const float* w, void* y, int ty, int ldy,
-                                     int rows, int D, int groups, float eps, int add, float woff, fls_stream_t s) {
+                                     int rows, int D, int groups, float eps, int add, float woff, int w_one, fls_stream_t s) {
   if (rows <= 0) return 0;
   if (groups < 1 || D % groups) return -1;
   dim3 grid(rows, groups);
   hipStream_t st = (hipStream_t)s;
-  if (add) hipLaunchKernelGGL((group_rmsnorm_kernel<float, 1>), grid, dim3(256), 0, st, x, ldx, idx, w, (float*)y, ldy, D, groups, eps, woff);
-  else if (ty == 1) hipLaunchKernelGGL((group_rmsnorm_kernel<bf16_t, 0>), grid, dim3(256), 0, st, x, ldx, idx, w, (bf16_t*)y, ldy, D, groups, eps, woff);
-  else hipLaunchKernelGGL((group_rmsnorm_kernel<float, 0>), grid, dim3(256), 0, st, x, ldx, idx, w, (float*)y, ldy, D, groups, eps, woff);
+  if (add) hipLaunchKernelGGL((group_rmsnorm_kernel<float, 1>), grid, dim3(256), 0, st, x, ldx, idx, w, (float*)y, ldy, D, groups, eps, woff, w_one);
+  else if (ty == 1) hipLaunchKernelGGL((group_rmsnorm_kernel<bf16_t, 0>), grid, dim3(256), 0, st, x, ldx, idx, w, (bf16_t*)y, ldy, D, groups, eps, woff, w_one);
+  else hipLaunchKernelGGL((group_rmsnorm_kernel<float, 0>), grid, dim3(256), 0, st, x, ldx, idx, w, (float*)y, ldy, D, groups, eps, woff, w_one);
   SEQ_LAUNCH_CHECK();
   return 0;
 }
@@ -664,4 +664,4 @@ extern "C" int fls_seq_moe_combine(float* x, int ldx, const float* y, int ldy, c
   return 0;
 }
 
-extern "C" int fls_seq_version(void) { return 10; }
+extern "C" int fls_seq_version(void) { return 11; }

@@ -147,9 +147,45 @@ extern "C" int fls_seq_causal_conv(const float* x, int ldx, const float* w, cons
 // row's heads), the four waves taking heads in turn; the host gives a row one block when rows are many and a wave
 // per head when they are few.  fuse_state (every request brings one row): the wave also rewrites its channels of
 // the carried history.  Head sizes <= 512.
+// half: the pairs are (i, i + rot / 2) instead (the other entry comes from whichever lane and register holds it); amp:
+// a factor on every cosine and sine; no_norm: q and k heads are only rotated.  pool.P > 0 (with fuse_state: every
+// request brings one row): the wave whose row completes a block of pool.P positions also writes the block's mean key
+// (value) -- the mean of the rows as the pages hold them, summed in position order -- to its row of the block pools.
 // TAPS > 0: that many taps, all of a head's inputs and weights loaded before the sums (the loads of a head are
 // in flight together); TAPS = 0: any number, or none.  NE: entries per lane (head sizes <= 64 NE).
 #define QKV_MAX_E 8
+struct BlockPools {
+  const int* page_table;     // [B, pt_stride]: pages of the rows
+  int pt_stride, page_size;
+  int P;                     // positions per block (0: no blocks)
+  void* kp;                  // block pools, rows ldkp / ldvp wide
+  int ldkp;
+  void* vp;
+  int ldvp;
+  const int* table;          // [B, t_stride]: pages of the blocks, page_size blocks each
+  int t_stride;
+};
+
+// the mean of column c over the P rows of block b of request s: positions b P .. b P + P - 1 of pool `src`, all but the
+// last from memory, the last one as given (or from memory too, last == nullptr)
+template <typename T>
+__device__ __forceinline__ float block_mean(const T* src, int ld, int c, const BlockPools& bp, int s, int b, const float* last) {
+  const int* tab = bp.page_table + (size_t)s * bp.pt_stride;
+  float acc = 0.f;
+  const int n = last != nullptr ? bp.P - 1 : bp.P;
+  for (int x = 0; x < n; ++x) {
+    const int j = b * bp.P + x;
+    acc += ldf(src + ((size_t)tab[j / bp.page_size] * bp.page_size + j % bp.page_size) * ld, c);
+  }
+  if (last != nullptr) acc += *last;
+  return acc / (float)bp.P;
+}
+__device__ __forceinline__ size_t block_row(const BlockPools& bp, int s, int b) {
+  return (size_t)bp.table[(size_t)s * bp.t_stride + b / bp.page_size] * bp.page_size + b % bp.page_size;
+}
+__device__ __forceinline__ float as_stored(const float*, float v) { return v; }
+__device__ __forceinline__ float as_stored(const bf16_t*, float v) { return bf16_to_f(f_to_bf16(v)); }
+
 template <typename TO, int TAPS, int NE>
 __global__ __launch_bounds__(256) void qkv_conv_rope_kernel(const float* __restrict__ z, int ldz, const float* __restrict__ w,
                                                             float* __restrict__ state, int taps, const int* __restrict__ tok_seq,
@@ -159,7 +195,8 @@ __global__ __launch_bounds__(256) void qkv_conv_rope_kernel(const float* __restr
                                                             const float* __restrict__ freqs, int rot, float* __restrict__ qo,
                                                             int ldq, TO* __restrict__ kc, int ldk, TO* __restrict__ vc, int ldv,
                                                             int C, int fuse_state, int Gv, const float* __restrict__ qnw,
-                                                            const float* __restrict__ knw) {
+                                                            const float* __restrict__ knw, int half, float amp, int no_norm,
+                                                            BlockPools pool) {
   const int lane = threadIdx.x & 63;
   const int t = blockIdx.x;
   const int ipr = H + G + Gv;
@@ -168,6 +205,7 @@ __global__ __launch_bounds__(256) void qkv_conv_rope_kernel(const float* __restr
   const bool carried = pos0[s] > 0;
   float* hist = (w != nullptr && taps > 1) ? state + (size_t)slot[s] * (taps - 1) * C : nullptr;
   float cs[NE], sn[NE];
+  const int hr = rot >> 1;
   {
     const float pos = rot > 0 ? (float)tok_pos[t] : 0.f;
 #pragma unroll
@@ -175,9 +213,15 @@ __global__ __launch_bounds__(256) void qkv_conv_rope_kernel(const float* __restr
       const int c = lane + 64 * e;
       cs[e] = 1.f;
       sn[e] = 0.f;
-      if (c < rot) sincosf(pos * freqs[c >> 1], &sn[e], &cs[e]);
+      if (c < rot) {
+        sincosf(pos * freqs[half ? (c >= hr ? c - hr : c) : c >> 1], &sn[e], &cs[e]);
+        cs[e] *= amp;
+        sn[e] *= amp;
+      }
     }
   }
+  // the block this row completes, if any (block-uniform)
+  const int blk = (fuse_state && pool.P > 0 && (tok_pos[t] + 1) % pool.P == 0) ? tok_pos[t] / pool.P : -1;
   for (int hi = blockIdx.y * 4 + (threadIdx.x >> 6); hi < ipr; hi += 4 * gridDim.y) {
     const int kind = hi < H ? 0 : (hi < H + G ? 1 : 2);
     const int n = kind == 2 ? dv : d;
@@ -240,6 +284,15 @@ __global__ __launch_bounds__(256) void qkv_conv_rope_kernel(const float* __restr
       TO* vr = vc + (size_t)kv_slot[t] * ldv + (size_t)(hi - H - G) * dv;
 #pragma unroll
       for (int e = 0; e < NE; ++e) { const int c = lane + 64 * e; if (c < n) stf(vr, c, v[e]); }
+      if (blk >= 0) {
+        TO* pr = reinterpret_cast<TO*>(pool.vp) + block_row(pool, s, blk) * pool.ldvp;
+#pragma unroll
+        for (int e = 0; e < NE; ++e) {
+          const int c = lane + 64 * e, col = (hi - H - G) * dv + c;
+          const float last = as_stored(vc, v[e]);
+          if (c < n) stf(pr, col, block_mean<TO>(vc, ldv, col, pool, s, blk, &last));
+        }
+      }
       continue;
     }
     float s2 = 0.f;
@@ -254,14 +307,37 @@ __global__ __launch_bounds__(256) void qkv_conv_rope_kernel(const float* __restr
         v[e] *= c < n ? nw[c] : 0.f;
       }
     }
+    float oth[NE];
+    if (half) {
+      if (NE == 2 && hr == 64) {                      // (the pair's other entry is this lane's other register)
+#pragma unroll
+        for (int e = 0; e < NE; ++e) oth[e] = v[NE - 1 - e];
+      } else {
+#pragma unroll
+        for (int e = 0; e < NE; ++e) {
+          const int c = lane + 64 * e;
+          const int pc = c < rot ? (c >= hr ? c - hr : c + hr) : c;
+          float o = 0.f;
+#pragma unroll
+          for (int e2 = 0; e2 < NE; ++e2) {
+            const float x = __shfl(v[e2], pc & 63, 64);
+            if ((pc >> 6) == e2) o = x;
+          }
+          oth[e] = o;
+        }
+      }
+    } else {
+#pragma unroll
+      for (int e = 0; e < NE; ++e) oth[e] = __shfl_xor(v[e], 1, 64);
+    }
 #pragma unroll
     for (int e = 0; e < NE; ++e) {
       const int c = lane + 64 * e;
-      const float other = __shfl_xor(v[e], 1, 64);
-      if (c < rot) v[e] = (c & 1) ? v[e] * cs[e] + other * sn[e] : v[e] * cs[e] - other * sn[e];
+      const bool second = half ? c >= hr : (c & 1);
+      if (c < rot) v[e] = second ? v[e] * cs[e] + oth[e] * sn[e] : v[e] * cs[e] - oth[e] * sn[e];
       if (nw == nullptr) s2 += v[e] * v[e];           // (entries past n are zeros)
     }
-    const float rs = 1.f / sqrtf(wave_sum(s2) / (float)n + eps);
+    const float rs = no_norm ? 1.f : 1.f / sqrtf(wave_sum(s2) / (float)n + eps);
     if (kind == 0) {
       float* qr = qo + (size_t)t * ldq + (size_t)hi * d;
 #pragma unroll
@@ -270,6 +346,15 @@ __global__ __launch_bounds__(256) void qkv_conv_rope_kernel(const float* __restr
       TO* kr = kc + (size_t)kv_slot[t] * ldk + (size_t)(hi - H) * d;
 #pragma unroll
       for (int e = 0; e < NE; ++e) { const int c = lane + 64 * e; if (c < n) stf(kr, c, v[e] * rs); }
+      if (blk >= 0) {
+        TO* pr = reinterpret_cast<TO*>(pool.kp) + block_row(pool, s, blk) * pool.ldkp;
+#pragma unroll
+        for (int e = 0; e < NE; ++e) {
+          const int c = lane + 64 * e, col = (hi - H) * d + c;
+          const float last = as_stored(kc, v[e] * rs);
+          if (c < n) stf(pr, col, block_mean<TO>(kc, ldk, col, pool, s, blk, &last));
+        }
+      }
     }
   }
 }
@@ -278,10 +363,11 @@ template <typename TO>
 static void qkv_launch(int TP, int ne, dim3 grid, hipStream_t st, const float* z, int ldz, const float* w, float* state, int taps,
                        const int* tok_seq, const int* tok_pos, const int* cu, const int* pos0, const int* slot, const int* kv_slot,
                        int H, int G, int d, int dv, float eps, const float* freqs, int rot, float* qo, int ldq, TO* kc, int ldk,
-                       TO* vc, int ldv, int C, int fuse, int Gv, const float* qnw, const float* knw) {
+                       TO* vc, int ldv, int C, int fuse, int Gv, const float* qnw, const float* knw, int half, float amp,
+                       int no_norm, const BlockPools& pool) {
 #define QKV_GO(TT, NN) hipLaunchKernelGGL((qkv_conv_rope_kernel<TO, TT, NN>), grid, dim3(256), 0, st, z, ldz, w, state, taps, tok_seq, \
                                           tok_pos, cu, pos0, slot, kv_slot, H, G, d, dv, eps, freqs, rot, qo, ldq, kc, ldk, vc, ldv, C, fuse, \
-                                          Gv, qnw, knw)
+                                          Gv, qnw, knw, half, amp, no_norm, pool)
 #define QKV_NE(TT) do { if (ne <= 1) QKV_GO(TT, 1); else if (ne <= 2) QKV_GO(TT, 2); else QKV_GO(TT, QKV_MAX_E); } while (0)
   if (TP == 2) QKV_NE(2);
   else if (TP == 3) QKV_NE(3);
@@ -295,7 +381,9 @@ extern "C" int fls_seq_qkv_conv_rope(const float* z, int ldz, const float* w, fl
                                      const int* tok_pos, const int* cu, const int* pos0, const int* slot, const int* kv_slot,
                                      int T, int B, int H, int G, int d, int dv, float eps, const float* freqs, int rot, float* qo,
                                      int ldq, void* kc, int ldk, void* vc, int ldv, int tc, int one_row_each, int Gv,
-                                     const float* qnw, const float* knw, fls_stream_t s) {
+                                     const float* qnw, const float* knw, int half, float amp, int no_norm,
+                                     const int* page_table, int pt_stride, int page_size, int P, void* kp, int ldkp, void* vp,
+                                     int ldvp, const int* block_table, int bt_stride, fls_stream_t s) {
   if (T <= 0) return 0;
   if (Gv < 0 || G == 0) Gv = G;
   if (H < 1 || G < 0 || d < 1 || d > 64 * QKV_MAX_E || dv > 64 * QKV_MAX_E || rot < 0 || rot > d || (rot & 1) ||
@@ -304,6 +392,11 @@ extern "C" int fls_seq_qkv_conv_rope(const float* z, int ldz, const float* w, fl
     return -1;
   const int C = H * d + G * d + Gv * dv;
   if (C > ldz || H * d > ldq || (G > 0 && (G * d > ldk || Gv * dv > ldv))) return -1;
+  if (no_norm && (qnw != nullptr || knw != nullptr)) return -1;
+  if (P < 0 || (P > 0 && (G < 1 || !one_row_each || T != B || page_size < 1 || page_table == nullptr || block_table == nullptr ||
+                          kp == nullptr || vp == nullptr || G * d > ldkp || Gv * dv > ldvp)))
+    return -1;
+  const BlockPools pool = {page_table, pt_stride, page_size, P, kp, ldkp, vp, ldvp, block_table, bt_stride};
   const int ipr = H + G + Gv;
   // blocks per row: one when the rows alone fill the chip (every wave then reuses its sines and cosines for a
   // quarter of the row's heads), up to a wave per head when rows are few
@@ -315,13 +408,77 @@ extern "C" int fls_seq_qkv_conv_rope(const float* z, int ldz, const float* w, fl
   hipStream_t st = (hipStream_t)s;
   const int TP = (w != nullptr && taps >= 2 && taps <= 4) ? taps : 0;
   const int ne = ((d > dv ? d : dv) + 63) / 64;
-  if (tc == 1) qkv_launch<bf16_t>(TP, ne, grid, st, z, ldz, w, state, taps, tok_seq, tok_pos, cu, pos0, slot, kv_slot, H, G, d, dv, eps, freqs, rot, qo, ldq, (bf16_t*)kc, ldk, (bf16_t*)vc, ldv, C, fuse, Gv, qnw, knw);
-  else qkv_launch<float>(TP, ne, grid, st, z, ldz, w, state, taps, tok_seq, tok_pos, cu, pos0, slot, kv_slot, H, G, d, dv, eps, freqs, rot, qo, ldq, (float*)kc, ldk, (float*)vc, ldv, C, fuse, Gv, qnw, knw);
+  if (tc == 1) qkv_launch<bf16_t>(TP, ne, grid, st, z, ldz, w, state, taps, tok_seq, tok_pos, cu, pos0, slot, kv_slot, H, G, d, dv, eps, freqs, rot, qo, ldq, (bf16_t*)kc, ldk, (bf16_t*)vc, ldv, C, fuse, Gv, qnw, knw, half, amp, no_norm, pool);
+  else qkv_launch<float>(TP, ne, grid, st, z, ldz, w, state, taps, tok_seq, tok_pos, cu, pos0, slot, kv_slot, H, G, d, dv, eps, freqs, rot, qo, ldq, (float*)kc, ldk, (float*)vc, ldv, C, fuse, Gv, qnw, knw, half, amp, no_norm, pool);
   SEQ_LAUNCH_CHECK();
   if (w != nullptr && taps > 1 && !fuse) {
     hipLaunchKernelGGL(conv_state_kernel, dim3((C + 255) / 256, B), dim3(256), 0, st, z, ldz, state, cu, pos0, slot, C, taps);
     SEQ_LAUNCH_CHECK();
   }
+  return 0;
+}
+
+// ------------------------------------------------------------------- means of key / value blocks
+// Block b of a request holds positions b P .. b P + P - 1; its mean key and mean value (the mean of the rows as the
+// page pools hold them, fp32 sums in position order) are rows of the block pools.  Grid: (column pieces, blocks a
+// request's rows of this step can complete, requests); a workgroup whose block is not completed by this step ends at
+// once.  A thread owns VE neighbouring columns of [keys | values] and walks the block's P rows.
+template <typename T, int VE>
+__global__ __launch_bounds__(256) void block_means_kernel(const T* __restrict__ kc, int ldk, const T* __restrict__ vc, int ldv,
+                                                          const int* __restrict__ cu, const int* __restrict__ pos0, int kcols,
+                                                          int vcols, BlockPools bp) {
+  const int s = blockIdx.z;
+  const int p0 = pos0[s], n = cu[s + 1] - cu[s];
+  const int b = p0 / bp.P + blockIdx.y;
+  if ((b + 1) * bp.P > p0 + n) return;
+  const int c0 = (blockIdx.x * 256 + threadIdx.x) * VE;
+  if (c0 >= kcols + vcols) return;
+  const bool isk = c0 < kcols;                       // (VE divides kcols)
+  const T* src = isk ? kc + c0 : vc + (c0 - kcols);
+  const int ld = isk ? ldk : ldv;
+  const int* tab = bp.page_table + (size_t)s * bp.pt_stride;
+  float acc[VE];
+#pragma unroll
+  for (int i = 0; i < VE; ++i) acc[i] = 0.f;
+  for (int x = 0; x < bp.P; ++x) {
+    const int j = b * bp.P + x;
+    const T* row = src + ((size_t)tab[j / bp.page_size] * bp.page_size + j % bp.page_size) * ld;
+    if constexpr (VE == 4 && sizeof(T) == 2) {
+      const uint2 v = *reinterpret_cast<const uint2*>(row);
+      const bf16_t* e = reinterpret_cast<const bf16_t*>(&v);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[i] += bf16_to_f(e[i]);
+    } else if constexpr (VE == 4) {
+      const float4 v = *reinterpret_cast<const float4*>(row);
+      acc[0] += v.x; acc[1] += v.y; acc[2] += v.z; acc[3] += v.w;
+    } else {
+      acc[0] += ldf(row, 0);
+    }
+  }
+  T* dst = (isk ? reinterpret_cast<T*>(bp.kp) + block_row(bp, s, b) * bp.ldkp + c0
+                : reinterpret_cast<T*>(bp.vp) + block_row(bp, s, b) * bp.ldvp + (c0 - kcols));
+#pragma unroll
+  for (int i = 0; i < VE; ++i) stf(dst, i, acc[i] / (float)bp.P);
+}
+
+extern "C" int fls_seq_block_means(const void* kc, int ldk, const void* vc, int ldv, int tc, const int* cu, const int* pos0, int B,
+                                   int max_rows, int kcols, int vcols, const int* page_table, int pt_stride, int page_size, int P,
+                                   void* kp, int ldkp, void* vp, int ldvp, const int* block_table, int bt_stride, fls_stream_t s) {
+  if (B <= 0 || max_rows <= 0) return 0;
+  if (P < 1 || page_size < 1 || kcols < 1 || vcols < 1 || kcols > ldk || vcols > ldv || kcols > ldkp || vcols > ldvp) return -1;
+  const BlockPools bp = {page_table, pt_stride, page_size, P, kp, ldkp, vp, ldvp, block_table, bt_stride};
+  const int es = tc == 1 ? 2 : 4;
+  auto al = [&](const void* p, int ld) { return (uintptr_t)p % (4 * es) == 0 && ld % 4 == 0; };
+  const int ve = (kcols % 4 == 0 && vcols % 4 == 0 && al(kc, ldk) && al(vc, ldv) && al(kp, ldkp) && al(vp, ldvp)) ? 4 : 1;
+  // n rows complete at most ceil(n / P) blocks
+  dim3 grid((kcols + vcols + 256 * ve - 1) / (256 * ve), (max_rows + P - 1) / P, B);
+  hipStream_t st = (hipStream_t)s;
+#define BM_GO(TT, VV) hipLaunchKernelGGL((block_means_kernel<TT, VV>), grid, dim3(256), 0, st, (const TT*)kc, ldk, (const TT*)vc, ldv, cu, \
+                                         pos0, kcols, vcols, bp)
+  if (tc == 1) { if (ve == 4) BM_GO(bf16_t, 4); else BM_GO(bf16_t, 1); }
+  else { if (ve == 4) BM_GO(float, 4); else BM_GO(float, 1); }
+#undef BM_GO
+  SEQ_LAUNCH_CHECK();
   return 0;
 }
 

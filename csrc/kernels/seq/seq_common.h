@@ -43,6 +43,18 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
   return z / (1.f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
 }
 
+// pooled blocks beside an attention window: one mean key and value for each block of P positions, rows of the block
+// pools kp / vp (rows ldk / ldv wide, pages of the attention's page size, table[request][t_stride])
+struct AttnBlocks {
+  int P;
+  const void* kp;
+  int ldk;
+  const void* vp;
+  int ldv;
+  const int* table;
+  int t_stride;
+};
+
 // attn_paged.hip: out[t, h] from nsplit partial (maximum, sum, weighted values) records per (row, head)
 typedef void* fls_stream_t;
 // has_sink: the softmax's silent entry of score `sink` joins the total here; head_gate (nullable) [T, H]: a sigmoid gate per (row, head)

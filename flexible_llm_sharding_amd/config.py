@@ -871,8 +871,104 @@ class LopilixConfig:
         return d
 
 
+@dataclass
+class NudadraConfig:
+    """Nudadra: a decoder whose layers run two mixers and a feed-forward side by side on one normed row,
+    x <- x + (rms(left(h)) w_l + rms(right(h)) w_r) / 2 + ff(h), h = g rms(x) with one number g per layer.
+    Left: grouped-query attention, rotated in pairs (i, i + dims / 2) with frequencies rescaled by how often
+    an entry turns over the original context; a query sees its window's tokens and, in the same softmax, the
+    mean key and value of every earlier block of ``mask.pool`` tokens; a sigmoid gate per head.  Right: a
+    Mamba-2 state-space mixer.  Feed-forward: squared-ReLU dense.  ``loop``: layers start .. stop - 1 run
+    ``times`` times in a row on the same weights; every pass starts from W_in [x; x0] + step_t, x0 the
+    embedding row, and has pages and states of its own (its layers are names of their own, ``l0@1``).
+    Everything is read from config.json: ``width``, ``vocab``, ``norm.eps``, ``embedding.scale``, ``loop``
+    and ``layers`` (per layer ``type``, ``mixer.left``, ``mixer.right``, ``mlp``)."""
+    width: int
+    vocab: int
+    norm_eps: float
+    embedding_scale: float
+    loop: Optional[dict]
+    layers: list
+    family = "nudadra"
+    model_type = "nudadra"
+    is_moe = False
+    sliding_window = None
+    tie_word_embeddings = False
+
+    hidden_size = KagolixConfig.hidden_size
+    vocab_size = KagolixConfig.vocab_size
+    save = KagolixConfig.save
+    order = LopilixConfig.order
+    num_hidden_layers = LopilixConfig.num_hidden_layers
+    num_layers_total = LopilixConfig.num_layers_total
+    layer_names = LopilixConfig.layer_names
+    layer = LopilixConfig.layer
+
+    def total_params(self) -> int:
+        from .models.layout import layer_image, layer_layout_of
+        images = dict.fromkeys(layer_image(n) for n in self.layer_names())
+        return sum(sum(s.numel for s in layer_layout_of(self, n).slots) for n in images)
+
+    @property
+    def state_width(self) -> int:
+        """Columns of the activation that passes from layer to layer: the residual row, and beside it the embedding
+        row when a loop reads it again."""
+        return (2 if self.loop else 1) * self.width
+
+    def loop_pass(self, name: str) -> Optional[int]:
+        """The number of the pass that layer run ``name`` opens, or None."""
+        i, _, p = name[1:].partition("@")
+        return int(p or 0) if self.loop and int(i) == int(self.loop["start"]) else None
+
+    def validate(self) -> None:
+        lp = self.loop
+        if lp and not (0 <= int(lp["start"]) < int(lp["stop"]) <= len(self.layers) and int(lp["times"]) >= 1):
+            raise ValueError(f"loop {lp} does not fit {len(self.layers)} layers")
+        for i, l in enumerate(self.layers):
+            if l.type != "parallel":
+                raise NotImplementedError(f"layer {i}: mixer type {l.type!r}")
+            a, r = l.mixer["left"], l.mixer["right"]
+            if a["heads"] % a["kv_heads"]:
+                raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+            rot = a.get("rot")
+            if rot is not None and (int(rot["dims"]) > a["dim"] or int(rot["dims"]) % 2):
+                raise ValueError(f"layer {i}: rot.dims must be even and at most dim")
+            if int(a["mask"]["size"]) < 1 or int(a["mask"]["pool"]) < 1:
+                raise ValueError(f"layer {i}: mask {a['mask']}")
+            if max(int(a["dim"]), int(a["vdim"])) > 512:
+                # (a head stays in one wave's registers on its way into the pages, 8 value columns a lane in the attention)
+                raise NotImplementedError(f"layer {i}: attention head sizes above 512")
+            if r["heads"] % r["groups"] or (r["heads"] * r["vdim"]) % r["norm_groups"]:
+                raise ValueError(f"layer {i}: groups / norm_groups do not divide the heads / the inner width")
+            if int(r["conv"]) < 1:
+                raise ValueError(f"layer {i}: conv must be >= 1 taps")
+            if not 1 <= int(r["state"]) <= 256:
+                # (the scan keeps a value column's state rows in the registers of 16 lanes, 16 rows each)
+                raise NotImplementedError(f"layer {i}: a recurrent state of more than 256 rows per head")
+            if l.mlp is not None and l.mlp.get("kind", "dense") != "dense":
+                raise NotImplementedError(f"layer {i}: mlp kind {l.mlp['kind']!r}")
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "NudadraConfig":
+        layers = [HybridLayer(l["type"], json.loads(json.dumps(l["mixer"])),
+                              None if l.get("mlp") is None else json.loads(json.dumps(l["mlp"]))) for l in d["layers"]]
+        cfg = cls(int(d["width"]), int(d["vocab"]), float(d["norm"]["eps"]), float((d.get("embedding") or {}).get("scale", 1.0)),
+                  json.loads(json.dumps(d.get("loop"))) or None, layers)
+        cfg.validate()
+        return cfg
+
+    def to_dict(self) -> dict:
+        d = {"architecture": "Nudadra", "width": self.width, "vocab": self.vocab, "norm": {"eps": self.norm_eps},
+             "embedding": {"scale": self.embedding_scale},
+             "layers": [{"type": l.type, "mixer": l.mixer, "mlp": l.mlp} for l in self.layers]}
+        if self.loop:
+            d["loop"] = self.loop
+        return d
+
+
 # "architecture" of config.json -> config class of a stateful hybrid family
-ARCHITECTURES = {"Kagolix": KagolixConfig, "Sisavik": SisavikConfig, "Gizezen": GizezenConfig, "Lopilix": LopilixConfig}
+ARCHITECTURES = {"Kagolix": KagolixConfig, "Sisavik": SisavikConfig, "Gizezen": GizezenConfig, "Lopilix": LopilixConfig,
+                 "Nudadra": NudadraConfig}
 
 
 def load_config(model_path: str):

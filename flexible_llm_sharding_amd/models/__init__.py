@@ -17,4 +17,7 @@ def hybrid_family(cfg):
     if fam == "lopilix":
         from . import lopilix
         return lopilix
+    if fam == "nudadra":
+        from . import nudadra
+        return nudadra
     raise NotImplementedError(f"no hybrid family {fam!r}")

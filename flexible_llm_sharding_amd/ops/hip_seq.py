@@ -81,13 +81,14 @@ class HipSeqOps:
         _rows(x, "x", torch.float32)
         rows = x.shape[0] if row_idx is None else row_idx.numel()
         D = x.shape[1]
-        _vec(w, "w", D)
+        one = D != 1 and w.numel() == 1
+        _vec(w, "w", 1 if one else D)
         if row_idx is not None:
             _vec(row_idx, "row_idx", rows, torch.int32)
         y = torch.empty(rows, D, dtype=out_dtype, device=x.device)
         _chk(self.k.fls_seq_group_rmsnorm(x.data_ptr(), x.stride(0), row_idx.data_ptr() if row_idx is not None else None,
                                           w.data_ptr(), y.data_ptr(), _CODE[out_dtype], D, rows, D, groups, float(eps), 0,
-                                          float(w_offset), _stream()), "fls_seq_group_rmsnorm")
+                                          float(w_offset), 1 if one else 0, _stream()), "fls_seq_group_rmsnorm")
         return y
 
     def add_group_rmsnorm_(self, x, y, w, groups, eps, w_offset=0.0):
@@ -97,9 +98,37 @@ class HipSeqOps:
             raise ValueError("add_group_rmsnorm_: shapes differ")
         _vec(w, "w", x.shape[1])
         _chk(self.k.fls_seq_group_rmsnorm(y.data_ptr(), y.stride(0), None, w.data_ptr(), x.data_ptr(), 0, x.stride(0),
-                                          x.shape[0], x.shape[1], groups, float(eps), 1, float(w_offset), _stream()),
+                                          x.shape[0], x.shape[1], groups, float(eps), 1, float(w_offset), 0, _stream()),
              "fls_seq_group_rmsnorm")
         return x
+
+    def residual_branches_(self, x, branches=None, coef=1.0, add=None, keep=True, eps=0.0, norm_w=None, out_dtype=torch.float32):
+        _rows(x, "x", torch.float32)
+        T, D = x.shape
+        a = wa = b = wb = h = None
+        if branches is not None:
+            (a, wa), (b, wb) = branches
+            for nme, t in (("a", a), ("b", b)):
+                _rows(t, nme, torch.float32)
+                if tuple(t.shape) != (T, D):
+                    raise ValueError("residual_branches_: a branch is shaped unlike x")
+            _vec(wa, "wa", D)
+            _vec(wb, "wb", D)
+        if add is not None:
+            _rows(add, "add", torch.float32)
+            if tuple(add.shape) != (T, D):
+                raise ValueError("residual_branches_: add is shaped unlike x")
+        one = 0
+        if norm_w is not None:
+            one = 1 if D != 1 and norm_w.numel() == 1 else 0
+            _vec(norm_w, "norm_w", 1 if one else D)
+            h = torch.empty(T, D, dtype=out_dtype, device=x.device)
+        ptr = lambda t: t.data_ptr() if t is not None else None
+        ld = lambda t: t.stride(0) if t is not None else 0
+        _chk(self.k.fls_seq_residual_branches(x.data_ptr(), x.stride(0), 1 if keep else 0, ptr(a), ld(a), ptr(wa), ptr(b), ld(b),
+                                              ptr(wb), float(coef), ptr(add), ld(add), ptr(h), _CODE[out_dtype], D, ptr(norm_w),
+                                              one, T, D, float(eps), _stream()), "fls_seq_residual_branches")
+        return h
 
     def dyt_norm(self, x, wb, alpha, out_dtype, row_idx=None):
         _rows(x, "x", torch.float32)
@@ -255,8 +284,32 @@ class HipSeqOps:
              "fls_seq_moe_place")
         return SeqRoute(ids, w, offs, rows, dest, top)
 
+    @staticmethod
+    def _block_args(blocks, kcols, vcols, page_size, dtype, B):
+        """(P, kp, ldkp, vp, ldvp, table, table stride) of ``blocks`` = (block keys, block values, table, P) for a kernel."""
+        if blocks is None:
+            return 0, None, 0, None, 0, None, 0
+        kp, vp, table, P = blocks
+        if kp.dtype != dtype or vp.dtype != dtype or not kp.is_contiguous() or not vp.is_contiguous() or kp.shape[1] != page_size \
+                or vp.shape[1] != page_size or kp.shape[-1] < kcols or vp.shape[-1] < vcols or int(P) < 1:
+            raise ValueError("blocks: the block pools do not fit the key / value pools")
+        if table.dtype != torch.int32 or table.dim() != 2 or table.shape[0] != B or table.stride(1) != 1:
+            raise TypeError("blocks: the table is an int32 [requests, pages] tensor")
+        return int(P), kp.data_ptr(), kp.shape[-1], vp.data_ptr(), vp.shape[-1], table.data_ptr(), table.stride(0)
+
+    def block_means(self, kc, vc, blocks, meta, kcols, vcols):
+        table = meta["page_table"]
+        if kc.dtype != vc.dtype or not kc.is_contiguous() or not vc.is_contiguous() or kcols > kc.shape[-1] or vcols > vc.shape[-1] \
+                or kc.shape[1] != vc.shape[1]:
+            raise ValueError("block_means: pools do not fit")
+        P, kp, ldkp, vp, ldvp, bt, bts = self._block_args(blocks, kcols, vcols, kc.shape[1], kc.dtype, meta["n_seqs"])
+        _chk(self.k.fls_seq_block_means(kc.data_ptr(), kc.shape[-1], vc.data_ptr(), vc.shape[-1], _code(kc, "kc"),
+                                        meta["cu"].data_ptr(), meta["pos0"].data_ptr(), meta["n_seqs"], int(meta["max_rows"]), kcols,
+                                        vcols, table.data_ptr(), table.stride(0), kc.shape[1], P, kp, ldkp, vp, ldvp, bt, bts,
+                                        _stream()), "fls_seq_block_means")
+
     def qkv_conv_rope_store(self, z, w, state, meta, H, G, d, dv, q_out, kc, vc, eps=0.0, rot=None, v_heads=None, q_norm=None,
-                            k_norm=None):
+                            k_norm=None, norm=True, half=False, blocks=None):
         _rows(z, "z", torch.float32)
         _rows(q_out, "q_out", torch.float32)
         T = z.shape[0]
@@ -283,10 +336,18 @@ class HipSeqOps:
                 raise ValueError("qkv_conv_rope_store: pools do not fit the head sizes")
             tc = _code(kc, "kc")
             _vec(meta["kv_slot"], "kv_slot", T, torch.int32)
-        dims, freqs = 0, None
+        dims, freqs, amp = 0, None, 1.0
         if rot is not None and rot[0] > 0:
+            from .torch_seq import TorchSeqOps
             dims = int(rot[0])
-            freqs = self.rope_freqs(dims, rot[1], z.device, rot[2] if len(rot) > 2 else None)
+            sc = rot[2] if len(rot) > 2 else None
+            freqs = self.rope_freqs(dims, rot[1], z.device, sc)
+            amp = TorchSeqOps.rope_amp(sc)
+        one_each = meta.get("max_rows") == 1
+        ptab = meta.get("page_table")
+        fused = blocks if one_each else None             # (a one-row step completes its blocks in the same launch)
+        if blocks is not None and not G:
+            raise ValueError("qkv_conv_rope_store: blocks belong to a layer with keys and values")
         _chk(self.k.fls_seq_qkv_conv_rope(z.data_ptr(), z.stride(0), w.data_ptr() if w is not None else None,
                                           state.data_ptr() if state is not None and taps > 1 else None, taps,
                                           meta["tok_seq"].data_ptr(), meta["tok_pos"].data_ptr(), meta["cu"].data_ptr(),
@@ -295,22 +356,28 @@ class HipSeqOps:
                                           freqs.data_ptr() if freqs is not None else None, dims, q_out.data_ptr(),
                                           q_out.stride(0), kc.data_ptr() if G else None, kc.shape[-1] if G else 0,
                                           vc.data_ptr() if G else None, vc.shape[-1] if G else 0, tc,
-                                          1 if meta.get("max_rows") == 1 else 0, Gv,
+                                          1 if one_each else 0, Gv,
                                           q_norm.data_ptr() if q_norm is not None else None,
-                                          k_norm.data_ptr() if k_norm is not None else None, _stream()), "fls_seq_qkv_conv_rope")
+                                          k_norm.data_ptr() if k_norm is not None else None, 1 if half else 0, float(amp),
+                                          0 if norm else 1, ptab.data_ptr() if fused is not None else None,
+                                          ptab.stride(0) if fused is not None else 0, kc.shape[1] if fused is not None else 0,
+                                          *self._block_args(fused, G * d, Gv * dv, kc.shape[1] if G else 0, kc.dtype if G else None,
+                                                            meta["n_seqs"]), _stream()), "fls_seq_qkv_conv_rope")
+        if blocks is not None and fused is None:
+            self.block_means(kc, vc, blocks, meta, G * d, Gv * dv)
         return q_out
 
     def _gemm(self, a, w, c, bias, M, N, K, lda, ldw, ldc, groups=1, offs=None, a_gs=0, a_mod=1, w_gs=0, c_gs=0,
-              act=None):
+              act=None, kind=0):
         _chk(self.k.fls_seq_gemm(a.data_ptr(), _code(a, "a"), w.data_ptr(), _code(w, "w"), c.data_ptr(), _code(c, "c"),
                                  bias.data_ptr() if bias is not None else None,
-                                 act.data_ptr() if act is not None else None, M, N, K, lda, ldw, ldc, groups,
+                                 act.data_ptr() if act is not None else None, kind, M, N, K, lda, ldw, ldc, groups,
                                  offs.data_ptr() if offs is not None else None, a_gs, a_mod, w_gs, c_gs, _stream()),
              "fls_seq_gemm")
 
-    def matmul_nt(self, a, w, bias=None, xielu=None, out_dtype=torch.float32):
-        """a . w^T (+ bias); ``xielu`` ({p, q}): that activation in the epilogue; ``out_dtype``: the
-        accumulator as it is (fp32) or rounded for the next product (bf16)."""
+    def matmul_nt(self, a, w, bias=None, xielu=None, out_dtype=torch.float32, relu2=False):
+        """a . w^T (+ bias); ``xielu`` ({p, q}) or ``relu2`` (max(z, 0)^2): that activation in the epilogue;
+        ``out_dtype``: the accumulator as it is (fp32) or rounded for the next product (bf16)."""
         _rows(a, "a")
         _rows(w, "w")
         M, K = a.shape
@@ -323,8 +390,11 @@ class HipSeqOps:
             _vec(bias, "bias", N)
         if xielu is not None:
             _vec(xielu, "xielu", 2)
+            if relu2:
+                raise ValueError("matmul_nt: one activation at a time")
         c = torch.empty(M, N, dtype=out_dtype, device=a.device)
-        self._gemm(a, w, c, bias, M, N, K, a.stride(0), w.stride(0), N, act=xielu)
+        self._gemm(a, w, c, bias, M, N, K, a.stride(0), w.stride(0), N, act=xielu,
+                   kind=1 if xielu is not None else (2 if relu2 else 0))
         return c
 
     def block_linear(self, u, w, b, blocks, cdt):
@@ -358,6 +428,7 @@ class HipSeqOps:
         return y
 
     _ACT = {"silu": 0, "gelu_tanh": 1}
+    POOL_TILE_SHAPES = ((128, 128), (96, 96), (64, 64), (32, 32), (128, 64), (64, 128))    # fls_seq_attn_prefill with blocks
     HEAD_TILE_SHAPES = ((576, 512), (320, 256), (192, 128))    # (key row, value columns) of fls_seq_attn_heads
 
     def gate_mul(self, gu, out_dtype, act="silu"):
@@ -474,7 +545,8 @@ class HipSeqOps:
                                      kcols, vcols, _stream()), "fls_seq_kv_store")
 
     def attn_paged(self, q, kcache, vcache, meta, H, G, d, dv, scale, softcap, r1, r2, chunk, page_size, out_dtype,
-                   window=0, keep_first=0, gate_bias=None, out_scale=1.0, out=None, sink=None, head_gate=None, v_heads=None):
+                   window=0, keep_first=0, gate_bias=None, out_scale=1.0, out=None, sink=None, head_gate=None, v_heads=None,
+                   blocks=None):
         _rows(q, "q")
         T = q.shape[0]
         if kcache.dtype != out_dtype or vcache.dtype != out_dtype or q.shape[1] != H * d \
@@ -507,8 +579,12 @@ class HipSeqOps:
             raise ValueError("attn_paged: a silent softmax entry and per-key sigmoid weights exclude each other")
         extra = (1 if sink is not None else 0, float(sink or 0.0), head_gate.data_ptr() if head_gate is not None else None,
                  head_gate.stride(0) if head_gate is not None else 0)
+        if blocks is not None and (window < 1 or chunk > 0 or keep_first or sink is not None or gate_bias is not None or r1 is not None):
+            raise ValueError("attn_paged: blocks go with a plain softmax over a window")
+        blk = self._block_args(blocks, G * d, Gv * dv, page_size, kcache.dtype, meta.get("n_seqs"))
         tiles = meta.get("q_tiles")
-        if tiles is not None and kcache.dtype == torch.bfloat16 and d in (64, 128) and dv in (64, 128):
+        if tiles is not None and kcache.dtype == torch.bfloat16 and (
+                (d in (64, 128) and dv in (64, 128)) if blocks is None else (d, dv) in self.POOL_TILE_SHAPES):
             # a step with many rows per request: the matrix-core kernel over row tiles
             rc = self.k.fls_seq_attn_prefill(q.data_ptr(), q.stride(0), _code(q, "q"), kcache.data_ptr(), ldk, vcache.data_ptr(),
                                              ldv, out.data_ptr(), to, out.stride(0), tiles.data_ptr(), tiles.shape[0],
@@ -517,7 +593,7 @@ class HipSeqOps:
                                              r1.data_ptr() if r1 is not None else None,
                                              r2.data_ptr() if r2 is not None else None, int(chunk), int(window),
                                              int(keep_first), gate_bias.data_ptr() if gate_bias is not None else None,
-                                             float(out_scale), int(page_size), *extra, Gv, _stream())
+                                             float(out_scale), int(page_size), *extra, Gv, *blk, _stream())
             if rc == 0:
                 return out
             if rc != -2:
@@ -526,9 +602,9 @@ class HipSeqOps:
         if chunk > 0:
             bound = min(bound, int(chunk))
         if window > 0:
-            bound = min(bound, int(window) + int(keep_first))
+            bound = min(bound, int(window) + int(keep_first) + (bound // blk[0] if blocks is not None else 0))
         if tiles is None and q.dtype == torch.float32 and kcache.dtype == torch.bfloat16 and gate_bias is None and r1 is None \
-                and sink is None and head_gate is None and softcap == 0 and chunk == 0 and H // G <= 32 and Gv == G and to == 1 \
+                and sink is None and head_gate is None and blocks is None and softcap == 0 and chunk == 0 and H // G <= 32 and Gv == G and to == 1 \
                 and (d, dv) in self.HEAD_TILE_SHAPES:
             # few rows whose heads share long key / value rows (decoding over cached latent rows): the heads of a
             # token as the columns of one matrix-core tile, every key tile staged once for all of them
@@ -554,7 +630,7 @@ class HipSeqOps:
                                        r2.data_ptr() if r2 is not None else None, int(chunk), int(window), int(keep_first),
                                        gate_bias.data_ptr() if gate_bias is not None else None, float(out_scale),
                                        int(page_size), nsplit, part.data_ptr() if part is not None else None, *extra, Gv,
-                                       _stream()), "fls_seq_attn_paged")
+                                       *blk, _stream()), "fls_seq_attn_paged")
         return out
 
     # ------------------------------------------------------------ recurrences

@@ -44,7 +44,8 @@ class TorchSeqOps:
         return e
 
     def group_rmsnorm(self, x, w, groups, eps, out_dtype, row_idx=None, w_offset=0.0):
-        """``w_offset``: added to the weight (1.0 for weights stored around zero)."""
+        """``w_offset``: added to the weight (1.0 for weights stored around zero).  ``w`` of one element: one number
+        for all columns."""
         if row_idx is not None:
             x = x.index_select(0, row_idx.long())
         T, D = x.shape
@@ -55,6 +56,19 @@ class TorchSeqOps:
     def add_group_rmsnorm_(self, x, y, w, groups, eps, w_offset=0.0):
         x.add_(self.group_rmsnorm(y, w, groups, eps, torch.float32, w_offset=w_offset))
         return x
+
+    def residual_branches_(self, x, branches=None, coef=1.0, add=None, keep=True, eps=0.0, norm_w=None, out_dtype=torch.float32):
+        """x <- (x if ``keep``) + coef * (rms(a) * wa + rms(b) * wb) + add with ``branches`` = ((a, wa), (b, wb)); ``branches``
+        and ``add`` are optional.  ``norm_w`` (a vector, or one number): returns rms(new x) * norm_w as ``out_dtype``, in the
+        same pass over the row."""
+        new = x.clone() if keep else torch.zeros_like(x)
+        for a, w in branches or ():
+            a = a.float()
+            new += coef * (a * torch.rsqrt(a.pow(2).mean(-1, keepdim=True) + eps) * w.float())
+        if add is not None:
+            new += add.float()
+        x.copy_(new)
+        return None if norm_w is None else self.group_rmsnorm(x, norm_w, 1, eps, out_dtype)
 
     def dyt_norm(self, x, wb, alpha, out_dtype, row_idx=None):
         """Dynamic Tanh: tanh(alpha x) w + b elementwise, no statistics of the row; ``wb`` = [w; b] ([2, D]),
@@ -113,7 +127,7 @@ class TorchSeqOps:
         """o * sigmoid(g), element by element."""
         return (o.float() * torch.sigmoid(g.float())).to(out_dtype)
 
-    def matmul_nt(self, a, w, bias=None, xielu=None, out_dtype=torch.float32):
+    def matmul_nt(self, a, w, bias=None, xielu=None, out_dtype=torch.float32, relu2=False):
         if a.dtype != w.dtype:
             a = a.to(w.dtype)
         y = (a @ w.t()).float() if w.dtype == torch.float32 else (a.float() @ w.float().t())
@@ -121,6 +135,8 @@ class TorchSeqOps:
             y = y + bias.float()
         if xielu is not None:
             return self.xielu(y, xielu, out_dtype)
+        if relu2:
+            y = torch.relu(y).square()
         return y.to(out_dtype)
 
     def block_linear(self, u, w, b, blocks, cdt):
@@ -248,8 +264,24 @@ class TorchSeqOps:
                 raw[rows, out_col + h * out_hs:out_col + h * out_hs + n] = keep[:, h].to(raw.dtype)
         return out
 
+    def block_means(self, kc, vc, blocks, meta, kcols, vcols):
+        """``blocks`` = (block keys, block values, table, P): every block of P positions (b P .. b P + P - 1) that this
+        step's rows complete gets its mean key and mean value, over the rows as the pools hold them, written to row b of the
+        request's pages in the block pools (``table`` [requests, pages]; as many blocks a page as the pools have rows)."""
+        kp, vp, table, P = blocks
+        ps = kc.shape[1]
+        cu, pos0 = meta["cu_host"], meta["pos0_host"]
+        for s in range(len(pos0)):
+            p0, p1 = int(pos0[s]), int(pos0[s]) + int(cu[s + 1] - cu[s])
+            for b in range(p0 // P, p1 // P):
+                j = torch.arange(b * P, (b + 1) * P, device=kc.device)
+                rows = meta["page_table"][s].long()[j // ps] * ps + j % ps
+                at = int(table[s, b // ps]) * ps + b % ps
+                kp.view(-1, kp.shape[-1])[at, :kcols] = kc.view(-1, kc.shape[-1])[rows, :kcols].float().mean(0).to(kp.dtype)
+                vp.view(-1, vp.shape[-1])[at, :vcols] = vc.view(-1, vc.shape[-1])[rows, :vcols].float().mean(0).to(vp.dtype)
+
     def qkv_conv_rope_store(self, z, w, state, meta, H, G, d, dv, q_out, kc, vc, eps=0.0, rot=None, v_heads=None, q_norm=None,
-                            k_norm=None):
+                            k_norm=None, norm=True, half=False, blocks=None):
         """The projected rows z = [q (H d) | k (G d) | v (G dv) | ...] of a step on their way into attention:
         a short causal convolution per channel (``w`` [C, taps], no bias; the last taps - 1 rows of a request
         carried in ``state[slot]``, None for one tap), then for q and k heads the pair rotation ``rot`` and
@@ -257,7 +289,8 @@ class TorchSeqOps:
         ``q_out`` [T, H d] fp32, k and v to the rows ``kv_slot`` of their pools.  G = 0 (kc, vc None): a layer
         that reads another layer's keys and values has only queries.  ``v_heads``: the row holds that many value
         heads (instead of G) behind its G key heads.  ``q_norm`` / ``k_norm`` ([d]): the q / k heads are instead
-        RMS-normed before the rotation and multiplied by that weight."""
+        RMS-normed before the rotation and multiplied by that weight; ``norm`` False: they are only rotated.  ``half``: the
+        pairs are (i, i + dims / 2).  ``blocks``: ``block_means`` of the rows just written."""
         Gv = G if v_heads is None else int(v_heads)
         C = H * d + G * d + Gv * dv
         u = z[:, :C]
@@ -266,11 +299,13 @@ class TorchSeqOps:
                 u = self.causal_conv(u, w, None, state, meta)
             else:
                 u = u.float() * w.float()[:, 0]
-        self.head_norm_rope(u, H, d, 0, d, q_out, 0, d, meta, w=q_norm, eps=eps, rot=rot, unit_after=q_norm is None)
+        self.head_norm_rope(u, H, d, 0, d, q_out, 0, d, meta, w=q_norm, eps=eps, rot=rot, unit_after=norm and q_norm is None, half=half)
         if G:
             self.head_norm_rope(u, G, d, H * d, d, kc.view(-1, kc.shape[-1]), 0, d, meta, w=k_norm, eps=eps, rot=rot,
-                                unit_after=k_norm is None, row_map=meta["kv_slot"])
+                                unit_after=norm and k_norm is None, row_map=meta["kv_slot"], half=half)
             self.head_norm_rope(u, Gv, dv, (H + G) * d, dv, vc.view(-1, vc.shape[-1]), 0, dv, meta, row_map=meta["kv_slot"])
+            if blocks is not None:
+                self.block_means(kc, vc, blocks, meta, G * d, Gv * dv)
         return q_out
 
     def softcap_(self, z, cap):
@@ -289,7 +324,8 @@ class TorchSeqOps:
         vcache.view(-1, vcache.shape[-1]).index_copy_(0, kv_slot.long(), v.to(vcache.dtype))
 
     def attn_paged(self, q, kcache, vcache, meta, H, G, d, dv, scale, softcap, r1, r2, chunk, page_size, out_dtype,
-                   window=0, keep_first=0, gate_bias=None, out_scale=1.0, out=None, sink=None, head_gate=None, v_heads=None):
+                   window=0, keep_first=0, gate_bias=None, out_scale=1.0, out=None, sink=None, head_gate=None, v_heads=None,
+                   blocks=None):
         """Row i of a request sees the keys j <= i of its own chunk (``chunk`` > 0: floor(i / chunk) ==
         floor(j / chunk)) or window (``window`` > 0: j > i - window, and besides them the first
         ``keep_first`` keys of the sequence), read from the request's pages.  Head h of H reads key /
@@ -299,7 +335,9 @@ class TorchSeqOps:
         more entry of that score and no value, p_j = exp(s_j) / (exp(sink) + sum exp(s)).  ``head_gate``
         [T, H] fp32: head h's output of row t times sigmoid(head_gate[t, h]).  The result times ``out_scale``.
         ``v_heads`` (a divisor of G): the pool holds only that many value heads, key head g reads value
-        head g % v_heads (several score maps over the same values).  ``out`` may be fp32 over bf16 pools."""
+        head g % v_heads (several score maps over the same values).  ``out`` may be fp32 over bf16 pools.
+        ``blocks`` (with a window and a plain softmax) = (block keys, block values, table, P) as for ``block_means``: the same
+        softmax also runs over the mean key and value of every block of P positions that ends before the window."""
         T = q.shape[0]
         res = torch.empty(T, H * dv, dtype=torch.float32, device=q.device)
         kf = kcache.reshape(-1, kcache.shape[-1])[:, :G * d].reshape(-1, G, d)
@@ -320,6 +358,13 @@ class TorchSeqOps:
                 js = torch.cat([torch.arange(0, min(keep_first, lo), device=q.device), js])
             rows = table[seq[t]].long()[js // page_size] * page_size + js % page_size
             kk, vv = kf[rows].float(), vf[rows].float()            # [n, G, d]
+            if blocks is not None:
+                kp, vp, btab, P = blocks
+                b = torch.arange(max(0, i - window + 1) // P, device=q.device)      # (b + 1) P - 1 <= i - window
+                br = btab[seq[t]].long()[b // page_size] * page_size + b % page_size
+                kk = torch.cat([kp.reshape(-1, kp.shape[-1])[br, :G * d].reshape(-1, G, d).float(), kk])
+                vb = vp.reshape(-1, vp.shape[-1])[br, :Gv * dv].reshape(-1, Gv, dv).float()
+                vv = torch.cat([vb.repeat(1, G // Gv, 1), vv])
             s = torch.einsum("hd,nhd->hn", qf[t], kk.repeat_interleave(rep, 1)) * scale
             if softcap > 0:
                 s = softcap * torch.tanh(s / softcap)

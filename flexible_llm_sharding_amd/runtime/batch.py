@@ -455,6 +455,8 @@ class StepBatch:
     # [B, max_rows] int32, only when every request starts at position 0 in a step of many rows: the
     # packed row of each request's position, a page table (pages of one row) over the step's own rows
     local_table: Optional[np.ndarray] = None
+    # block length P -> [B, pages] int32 pages of the requests' key / value blocks (SequenceStateCache.block_table)
+    block_tables: dict = field(default_factory=dict)
     prompt_ids: List[int] = field(default_factory=lambda: [0])
     _dev: dict = field(default_factory=dict, repr=False)
 
@@ -481,6 +483,9 @@ class StepBatch:
             if self.local_table is not None:
                 names.append("local_table")
             arrs = [np.ascontiguousarray(getattr(self, k), dtype=np.int32) for k in names]
+            for P, t in self.block_tables.items():
+                names.append(f"block_table_{P}")
+                arrs.append(np.ascontiguousarray(t, dtype=np.int32))
             offs = np.cumsum([0] + [-(-a.size // 16) * 16 for a in arrs])
             flat = np.zeros(int(offs[-1]) + 16, dtype=np.int32)
             for a, o in zip(arrs, offs[:-1]):
@@ -531,7 +536,8 @@ def pack_step(entries: Sequence[StepEntry], cache) -> StepBatch:
                        for o in range(0, b - a, Q_TILE_ROWS)])
         tile_cu = i32(np.concatenate([[0], np.cumsum([-(-(b - a) // Q_TILE_ROWS) for a, b in zip(cu[:-1], cu[1:])])]))
     return StepBatch(rids, i32(ids), i32(seq), i32(pos), i32(cu), i32(pos0), i32(slot), table,
-                     i32(pages.astype(np.int64) * ps + pos_a % ps), i32(want), wc, len(ids), max_rows, q_tiles, tile_cu, local)
+                     i32(pages.astype(np.int64) * ps + pos_a % ps), i32(want), wc, len(ids), max_rows, q_tiles, tile_cu, local,
+                     {P: cache.block_table(rids, P) for P in cache.block_sizes})
 
 
 def split_step(entries: Sequence[StepEntry], token_budget: int) -> List[List[int]]:

@@ -240,7 +240,8 @@ class StepGraphs:
     A step mutates per-request state (K/V pages, recurrence slots), so there is no warm-up run: the
     first step of a shape runs eagerly (and does every lazy initialisation), the second is captured
     (capture executes nothing) and replayed, later ones only replayed.  The key is (requests in the
-    step, page-table width rounded up to ``TABLE_BUCKET`` pages, the state cache's generation): the
+    step, widths of the page table and of the block page tables rounded up to ``TABLE_BUCKET`` pages, the state
+    cache's generation): the
     pools' addresses are baked into the graph, so a pool that grew starts a new generation and the old
     graphs are dropped.  Every row's logits are computed (``want_idx`` = all rows); the caller picks
     the wanted ones."""
@@ -258,12 +259,18 @@ class StepGraphs:
         self.captures = self.replays = self.eager = 0
         self.generation = -1
 
-    def host_meta(self, batch, width: int) -> Dict[str, np.ndarray]:
+    @classmethod
+    def _widened(cls, t: np.ndarray) -> np.ndarray:
+        w = np.zeros((t.shape[0], _ceil(t.shape[1], cls.TABLE_BUCKET)), np.int32)
+        w[:, :t.shape[1]] = np.maximum(t, 0)
+        return w
+
+    def host_meta(self, batch) -> Dict[str, np.ndarray]:
         B = len(batch.rids)
-        table = np.zeros((B, width), np.int32)
-        table[:, :batch.page_table.shape[1]] = np.maximum(batch.page_table, 0)
         m = {k: getattr(batch, k) for k in self.KEYS if k not in ("page_table", "want_idx")}
-        m["page_table"] = table
+        m["page_table"] = self._widened(batch.page_table)
+        for P, t in batch.block_tables.items():
+            m[f"block_table_{P}"] = self._widened(t)
         m["want_idx"] = np.arange(B, dtype=np.int32)
         return m
 
@@ -274,9 +281,8 @@ class StepGraphs:
             self.seen.clear()
             self.generation = generation
         B = len(batch.rids)
-        width = _ceil(batch.page_table.shape[1], self.TABLE_BUCKET)
-        key = (B, width)
-        host = self.host_meta(batch, width)
+        host = self.host_meta(batch)
+        key = (B,) + tuple(v.shape[1] for v in host.values() if v.ndim == 2)
         g = self.graphs.get(key)
         if g is None:
             meta = {k: torch.from_numpy(np.ascontiguousarray(v)).to(self.dev) for k, v in host.items()}

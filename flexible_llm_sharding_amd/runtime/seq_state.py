@@ -9,6 +9,11 @@ The scoring engine's :class:`~.prefix_cache.PrefixKVCache` keeps whole prefixes 
   layer's pools instead of owning any.  A request holds a list of page numbers, the same in every
   layer's pool, so one page table serves all layers.  Token at position p of a request sits in row
   ``p % page_size`` of page ``table[p // page_size]``;
+* an attention layer that sees the tokens before its window as blocks of P positions owns block pools
+  besides, ``[block pages, page_size, width]``: the mean key and the mean value of every complete block.
+  A request's blocks have pages of their own (one list per P, whichever layers use it): block b sits in
+  row ``b % page_size`` of block page ``block_table[P][b // page_size]``.  They are kept for as long as the
+  request lives, also when the pages of the tokens they stand for have been given back;
 * every recurrent layer owns ``[slots, ...]`` fp32 tensors: the recurrence's state and the last
   ``taps - 1`` inputs of its short convolution.  A request holds one slot number, the same in every
   layer.  A request that starts at position 0 never reads its slot (the kernels start from zeros),
@@ -30,13 +35,14 @@ PAGE_SIZE = 16
 
 
 class _Request:
-    __slots__ = ("slot", "pages", "length", "first_page")
+    __slots__ = ("slot", "pages", "length", "first_page", "block_pages")
 
     def __init__(self, slot: int):
         self.slot = slot
         self.pages: List[int] = []     # page numbers from logical page ``first_page`` on (-1: given back)
         self.length = 0                # tokens stored so far
         self.first_page = 0
+        self.block_pages: Dict[int, List[int]] = {}      # block length P -> pages of the request's blocks
 
 
 class SequenceStateCache:
@@ -46,6 +52,7 @@ class SequenceStateCache:
         # what the model family keeps per request (models.hybrid_family(cfg).state_spec):
         #   paged    layer -> {pool: row width}: pools [pages, page_size, width] of the GEMM type
         #   alias    layer -> the layer whose pools it reads (a layer that shares another's keys)
+        #   blocks   layer -> (P, {pool: row width}): pools with one row per complete block of P positions
         #   slots    layer -> {tensor: shape}: fp32 [slots, *shape]
         #   horizons (kind, size, keep_first) of every layer that reads pages: "chunk": the keys of the
         #            current chunk of ``size`` positions; "window": the last ``size`` positions, and for
@@ -54,11 +61,18 @@ class SequenceStateCache:
         spec = hybrid_family(cfg).state_spec(cfg)
         self.attn: Dict[str, dict] = dict(spec["paged"])
         self.alias: Dict[str, str] = dict(spec.get("alias", {}))
+        self.blocks: Dict[str, tuple] = {k: (int(P), dict(w)) for k, (P, w) in spec.get("blocks", {}).items()}
+        self.block_sizes = sorted({P for P, _ in self.blocks.values()})
         self.rec: Dict[str, dict] = dict(spec["slots"])
         self.horizons = list(spec["horizons"])
         self.keep_pages = max([-(-int(k) // self.page_size) for _, _, k in self.horizons] + [0])
         self._kv: Dict[str, Dict[str, torch.Tensor]] = {}
         self._rec: Dict[str, Dict[str, torch.Tensor]] = {}
+        self._blk: Dict[str, Dict[str, torch.Tensor]] = {}
+        self.n_block_pages = {P: 0 for P in self.block_sizes}
+        self.free_block_pages: Dict[int, List[int]] = {P: [] for P in self.block_sizes}
+        self.block_pages_reused = 0
+        self._ever_block_pages = {P: set() for P in self.block_sizes}
         self.n_pages = self.n_slots = 0
         self.free_pages: List[int] = []
         self.free_slots: List[int] = []
@@ -68,6 +82,8 @@ class SequenceStateCache:
         self._ever_pages, self._ever_slots = set(), set()
         self._grow_pages(max(2, -(-int(max_tokens) // self.page_size) + int(max_seqs)))
         self._grow_slots(max(1, int(max_seqs)))
+        for P in self.block_sizes:
+            self._grow_block_pages(P, max(1, int(max_tokens) // (P * self.page_size) + int(max_seqs)))
 
     # ------------------------------------------------------------------ pools
     def _grow_pages(self, n: int) -> None:
@@ -81,6 +97,22 @@ class SequenceStateCache:
             self._kv[name] = new
         self.free_pages = list(range(n - 1, self.n_pages - 1, -1)) + self.free_pages
         self.n_pages = n
+        self.generation += 1
+
+    def _grow_block_pages(self, P: int, n: int) -> None:
+        old = self.n_block_pages[P]
+        if n <= old:
+            return
+        for name, (size, widths) in self.blocks.items():
+            if size != P:
+                continue
+            new = {k: torch.empty(n, self.page_size, w, dtype=self.dtype, device=self.dev) for k, w in widths.items()}
+            if name in self._blk:
+                for k in new:
+                    new[k][:old].copy_(self._blk[name][k])
+            self._blk[name] = new
+        self.free_block_pages[P] = list(range(n - 1, old - 1, -1)) + self.free_block_pages[P]
+        self.n_block_pages[P] = n
         self.generation += 1
 
     def _grow_slots(self, n: int) -> None:
@@ -104,11 +136,17 @@ class SequenceStateCache:
         p = self.pools(layer)
         return p["k"], p["v"]
 
+    def block_pools(self, layer: str, meta: dict) -> tuple:
+        """(block keys, block values, the step's block page table, P) of an attention layer with pooled blocks."""
+        P = self.blocks[layer][0]
+        p = self._blk[layer]
+        return p["k"], p["v"], meta[f"block_table_{P}"], P
+
     def recurrent(self, layer: str) -> Dict[str, torch.Tensor]:
         return self._rec[layer]
 
     def nbytes(self) -> int:
-        n = sum(t.numel() * t.element_size() for p in self._kv.values() for t in p.values())
+        n = sum(t.numel() * t.element_size() for pools in (self._kv, self._blk) for p in pools.values() for t in p.values())
         return n + sum(t.numel() * 4 for r in self._rec.values() for t in r.values())
 
     # --------------------------------------------------------------- requests
@@ -136,6 +174,16 @@ class SequenceStateCache:
             self.pages_reused += p in self._ever_pages
             self._ever_pages.add(p)
             r.pages.append(p)
+        for P in self.block_sizes:
+            mine, free = r.block_pages.setdefault(P, []), self.free_block_pages
+            need = -(-((pos0 + n_tokens) // P) // self.page_size)
+            while len(mine) < need:
+                if not free[P]:
+                    self._grow_block_pages(P, 2 * self.n_block_pages[P])
+                p = free[P].pop()
+                self.block_pages_reused += p in self._ever_block_pages[P]
+                self._ever_block_pages[P].add(p)
+                mine.append(p)
         r.length = pos0 + n_tokens
         return pos0, r.slot
 
@@ -169,6 +217,8 @@ class SequenceStateCache:
         if r is None:
             return
         self.free_pages += [p for p in r.pages if p >= 0]
+        for P, pages in r.block_pages.items():
+            self.free_block_pages[P] += pages
         self.free_slots.append(r.slot)
 
     def page_table(self, rids: Sequence) -> np.ndarray:
@@ -178,6 +228,15 @@ class SequenceStateCache:
         for j, i in enumerate(rids):
             r = self.requests[i]
             t[j, r.first_page:r.first_page + len(r.pages)] = r.pages
+        return t
+
+    def block_table(self, rids: Sequence, P: int) -> np.ndarray:
+        """[len(rids), widest] int32 pages of the requests' blocks of P positions (-1: none)."""
+        width = max([len(self.requests[i].block_pages.get(P, ())) for i in rids] + [1])
+        t = np.full((len(rids), width), -1, dtype=np.int32)
+        for j, i in enumerate(rids):
+            pages = self.requests[i].block_pages.get(P, ())
+            t[j, :len(pages)] = pages
         return t
 
     def live_tokens(self) -> int:
