@@ -1,7 +1,8 @@
 """Throughput of a hybrid stack next to the closest existing model at equal size: ``bench.py --hybrid``
 (Kagolix beside a Mixtral-structured stack; ``--hybrid-family sisavik``: Sisavik beside Kagolix;
 ``--hybrid-family gizezen``: Gizezen beside a Kagolix stack of attention layers with experts;
-``--hybrid-family lopilix``: Lopilix beside the Kagolix stack of attention, recurrent and state-space layers).
+``--hybrid-family lopilix``: Lopilix beside the Kagolix stack of attention, recurrent and state-space layers;
+``--hybrid-family nudadra``: Nudadra beside a Kagolix stack with the same mixers one after the other).
 
 Random weights at sizes that resemble a real model's layers.  Three parts, one JSON line each:
 
@@ -22,7 +23,7 @@ from typing import Dict, List
 import numpy as np
 import torch
 
-from ..config import GizezenConfig, KagolixConfig, LopilixConfig, ModelConfig, SisavikConfig
+from ..config import GizezenConfig, KagolixConfig, LopilixConfig, ModelConfig, NudadraConfig, SisavikConfig
 
 PEAK_FLOPS = 2.5e15        # dense bf16 / fp16 matrix peak of one MI355X
 PEAK_BYTES = 8.0e12        # HBM3E
@@ -117,6 +118,28 @@ def lopilix_config(z: dict, times: int = 2, streams: int = 4) -> LopilixConfig:
                                     "loop": {"start": 0, "stop": 3, "times": times}, "layers": layers})
 
 
+def nudadra_config(z: dict) -> NudadraConfig:
+    """Four layers, the middle two run twice in a row (six layer runs), each with windowed attention over tokens and
+    pooled blocks, a state-space mixer and a dense feed-forward side by side: head sizes, window and block length of
+    the order real models use."""
+    d = z["dim"]
+    left = {"heads": z["heads"], "kv_heads": z["kv"], "dim": d, "vdim": d, "scale": d ** -0.5, "mask": {"size": z["chunk"] // 2, "pool": 16},
+            "rot": {"dims": d, "base": 1.0e6, "scaling": {"factor": 4.0, "original": 4096, "fast": 24.0, "slow": 2.0}}}
+    right = {"heads": z["mh"], "vdim": z["mp"], "state": z["state"], "groups": 1, "norm_groups": 1, "conv": 4}
+    lay = {"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": {"kind": "dense", "ff": z["ff"]}}
+    return NudadraConfig.from_dict({"architecture": "Nudadra", "width": z["width"], "vocab": z["vocab"], "norm": {"eps": 1e-6},
+                                    "embedding": {"scale": 4.0}, "loop": {"start": 1, "stop": 3, "times": 2}, "layers": [lay] * 4})
+
+
+def kagolix_attention_mamba_config(z: dict, pairs: int = 6) -> KagolixConfig:
+    """The Kagolix stack a Nudadra stack is measured against: per layer run of that one an attention layer with a dense
+    feed-forward and a Mamba-2 layer without one, of the same sizes."""
+    cfg = hybrid_config(z, 1).to_dict()
+    att, _, mb = cfg["layers"]
+    cfg["layers"] = [att, dict(mb, mlp=None)] * pairs
+    return KagolixConfig.from_dict(cfg)
+
+
 def kagolix_attention_moe_config(z: dict, n_layers: int = 6) -> KagolixConfig:
     """The Kagolix stack a Gizezen stack is measured against: chunk-local attention and routed experts in
     every layer (the same heads, head size, experts and expert width; no shared expert, no shared keys)."""
@@ -160,7 +183,7 @@ def synthetic_hybrid_store(cfg: KagolixConfig, device, dtype, seed: int = 0):
                 v.copy_(0.9 * torch.rand(v.shape, generator=g, device=device))
             elif k.startswith("alpha"):
                 v.fill_(0.5)
-            elif k.startswith("norm") or k in ("qn", "kn", "mnorm", "dqn", "dkvn", "lqn", "lkn", "rnorm"):
+            elif k.startswith("norm") or k in ("outl", "outr", "qn", "kn", "mnorm", "dqn", "dkvn", "lqn", "lkn", "rnorm"):
                 v.copy_(1.0 + 0.1 * torch.randn(v.shape, generator=g, device=device))
             elif k in ("r1", "r2"):
                 v.copy_(torch.rand(v.shape, generator=g, device=device))       # (a negative r2 has no logarithm)
@@ -712,66 +735,150 @@ def bench_lopilix_kernels(z: dict, dtype, B: int, L: int, dev) -> dict:
     return {"part": "kernels", "family": "lopilix", "dtype": str(dtype), "batch": B, "context": L, "kernels": res}
 
 
+def bench_nudadra_kernels(z: dict, dtype, B: int, L: int, dev) -> dict:
+    """The kernels of a Nudadra layer alone at the prefill shape (T = B L rows) and the decode shape (B rows at context
+    L), each beside the like kernel of the Kagolix family on a like shape."""
+    from ..models.nudadra import BRANCH_WEIGHT, _cols, _rot
+    from ..ops import get_ops
+    ops = get_ops(dev, dtype, family="hybrid")
+    es = 2 if dtype == torch.bfloat16 else 4
+    cfg = nudadra_config(z)
+    mix, mlp = cfg.layers[0].mixer, cfg.layers[0].mlp
+    m, r = mix["left"], mix["right"]
+    D, ps = z["width"], 16
+    H, G, d, win, P = m["heads"], m["kv_heads"], m["dim"], m["mask"]["size"], m["mask"]["pool"]
+    c = _cols(mix)
+    res: Dict[str, dict] = {}
+
+    def rec(name, sec, flops=0.0, nbytes=0.0):
+        e = {"us": sec * 1e6}
+        if flops:
+            e["tflops"] = flops / sec / 1e12
+            e["of_matrix_peak"] = flops / sec / PEAK_FLOPS
+        if nbytes:
+            e["gb_s"] = nbytes / sec / 1e9
+            e["of_hbm"] = nbytes / sec / PEAK_BYTES
+        res[name] = {k: round(v, 4) for k, v in e.items()}
+
+    for tag, lens, pos0 in (("prefill", [L] * B, [0] * B), ("decode", [1] * B, [L - 1] * B)):
+        T = sum(lens)
+        meta = step_meta(B, lens, pos0, L, dev, ps)
+        meta["max_rows"] = max(lens)
+        pos = meta["pos_host"]
+        reps = 5 if tag == "prefill" else 30
+        nbp = -(-(L // P + 1) // ps)                     # block pages of a request
+        kc, vc = (torch.randn(meta["n_pages"], ps, G * d, device=dev).to(dtype) for _ in range(2))
+        kp, vp = (torch.randn(B * nbp, ps, G * d, device=dev).to(dtype) for _ in range(2))
+        blocks = (kp, vp, torch.arange(B * nbp, dtype=torch.int32, device=dev).view(B, nbp), P)
+        z_all = torch.randn(T, c["all"][1], device=dev)
+        col = lambda n: z_all[:, c[n][0]:c[n][0] + c[n][1]]
+        # attention over window and blocks | Kagolix: chunk-local softmax attention
+        q = torch.randn(T, H * d, device=dev)
+        keys = float(np.mean([min(p + 1, win) + max(0, p - win + 1) // P for p in pos]))
+        rec(f"{tag}/window + pooled blocks attention, head gates", _timed(lambda: ops.attn_paged(
+            q, kc, vc, meta, H, G, d, d, d ** -0.5, 0.0, None, None, 0, ps, dtype, window=win, blocks=blocks, head_gate=col("g")), reps),
+            4.0 * T * keys * H * d, 0 if tag == "prefill" else 2.0 * B * keys * G * d * es)
+        qk = q.to(dtype)
+        r1 = torch.rand(H, device=dev)
+        keys_k = float(np.mean([p % z["chunk"] + 1 for p in pos]))
+        rec(f"kagolix {tag}/chunk attention", _timed(lambda: ops.attn_paged(qk, kc, vc, meta, H, G, d, d, d ** -0.5, 30.0, r1, r1,
+                                                                              z["chunk"], ps, dtype), reps),
+            4.0 * T * keys_k * H * d, 0 if tag == "prefill" else 2.0 * B * keys_k * G * d * es)
+        # rotation of q and k, page write, block means | Kagolix: query norm, key norm + page write
+        C = (H + 2 * G) * d
+        qo = torch.empty(T, H * d, device=dev)
+        rot = _rot(m)
+
+        def qkv_path():
+            ops.qkv_conv_rope_store(z_all, None, None, meta, H, G, d, d, qo, kc, vc, rot=rot, norm=False, half=True, blocks=blocks)
+        means = T * 2 * G * d * es * (1.0 + 1.0 / P)     # (every row read back once, a mean written per block)
+        rec(f"{tag}/q k rotation, k v page write, block means", _timed(qkv_path, reps), 0,
+            T * (C * 4 + H * d * 4 + 2 * G * d * es) + means)
+        if tag == "prefill":
+            rec(f"{tag}/block means alone", _timed(lambda: ops.block_means(kc, vc, blocks, meta, G * d, G * d), reps), 0, means)
+        kn, qn = torch.ones(G * d, device=dev), torch.ones(H * d, device=dev)
+
+        def kagolix_qkv():
+            ops.group_rmsnorm(z_all[:, :H * d], qn, 1, 1e-6, out_dtype=dtype)
+            ops.kv_store(z_all[:, H * d:(H + G) * d], kn, 1e-6, z_all[:, (H + G) * d:C], kc, vc, meta["kv_slot"])
+        rec(f"kagolix {tag}/query norm, key norm + page write", _timed(kagolix_qkv, reps), 0, T * (C * 4 + (H + 2 * G) * d * es))
+        # the norm at the layer's start, the update at its end, the entry of a pass
+        x, ya, yb, ff = (torch.randn(T, 2 * D, device=dev)[:, :D] for _ in range(4))
+        nw, one = torch.ones(D, device=dev), torch.ones(1, device=dev)
+        rec(f"{tag}/norm with one number", _timed(lambda: ops.group_rmsnorm(x, one, 1, 1e-6, dtype), reps), 0, T * D * (4 + es))
+        rec(f"kagolix {tag}/group norm", _timed(lambda: ops.group_rmsnorm(x, nw, 2, 1e-6, dtype), reps), 0, T * D * (4 + es))
+        rec(f"{tag}/two branch norms + feed-forward + residual", _timed(lambda: ops.residual_branches_(
+            x, ((ya, nw), (yb, nw)), coef=BRANCH_WEIGHT, add=ff, eps=1e-6), reps), 0, T * D * 20)
+        rec(f"kagolix {tag}/post-norm + residual add", _timed(lambda: ops.add_group_rmsnorm_(x, ya, nw, 2, 1e-6), reps), 0, T * D * 12)
+        rec(f"{tag}/pass entry: row replaced + norm", _timed(lambda: ops.residual_branches_(
+            x, add=ya, keep=False, eps=1e-6, norm_w=one, out_dtype=dtype), reps), 0, T * D * (8 + es))
+        # the state-space side: the same convolution, scan and norm serve Kagolix
+        nh, vd, N = r["heads"], r["vdim"], r["state"]
+        cw, cb = torch.randn(c["xbc"][1], r["conv"], device=dev), torch.randn(c["xbc"][1], device=dev)
+        cst = torch.zeros(B, r["conv"] - 1, c["xbc"][1], device=dev)
+        rec(f"{tag}/causal convolution", _timed(lambda: ops.causal_conv(col("xbc"), cw, cb, cst, meta, act="silu"), reps), 0, T * c["xbc"][1] * 8)
+        xbc = torch.randn(T, c["xbc"][1], device=dev)
+        hp = torch.rand(nh, device=dev)
+        sst = torch.zeros(B, nh, N, vd, device=dev)
+        rec(f"{tag}/state-space scan", _timed(lambda: ops.ssd_scan(xbc, col("z"), col("dt"), hp, hp * 0.3, hp, sst, meta, nh, vd, N, 1), reps),
+            6.0 * T * nh * vd * N, (T * nh * vd * 12) if tag == "prefill" else 8.0 * B * nh * N * vd)
+        z2, dt = torch.randn(T, nh * vd, device=dev), torch.randn(T, nh, device=dev)
+        rec(f"kagolix {tag}/state-space scan", _timed(lambda: ops.ssd_scan(xbc, z2, dt, hp, hp * 0.3, hp, sst, meta, nh, vd, N, 1), reps),
+            6.0 * T * nh * vd * N, (T * nh * vd * 12) if tag == "prefill" else 8.0 * B * nh * N * vd)
+        # products
+        h = torch.randn(T, D, device=dev).to(dtype)
+        fw = int(mlp["ff"])
+        n_in = c["all"][1]
+        w = (0.02 * torch.randn(n_in, D, device=dev)).to(dtype)
+        rec(f"{tag}/gemm {T}x{n_in}x{D}", _timed(lambda: ops.matmul_nt(h, w), reps), 2.0 * T * n_in * D,
+            es * (n_in * D + T * D) + 4 * T * n_in)
+        wu = (0.02 * torch.randn(fw, D, device=dev)).to(dtype)
+        rec(f"{tag}/gemm {T}x{fw}x{D} + squared relu", _timed(lambda: ops.matmul_nt(h, wu, relu2=True, out_dtype=dtype), reps), 2.0 * T * fw * D,
+            es * (fw * D + T * D + T * fw))
+        act = torch.tensor([0.3, -0.2], device=dev)
+        rec(f"kagolix {tag}/gemm {T}x{fw}x{D} + xielu", _timed(lambda: ops.matmul_nt(h, wu, xielu=act, out_dtype=dtype), reps), 2.0 * T * fw * D,
+            es * (fw * D + T * D + T * fw))
+        wl = (0.02 * torch.randn(D, 2 * D, device=dev)).to(dtype)
+        xs, sv = torch.randn(T, 2 * D, device=dev), torch.randn(D, device=dev)
+        rec(f"{tag}/pass entry gemm {T}x{D}x{2 * D}, fp32 rows", _timed(lambda: ops.matmul_nt(xs, wl, bias=sv), reps), 4.0 * T * D * D,
+            es * 2 * D * D + 12 * T * D)
+        wk = (0.02 * torch.randn(D, 2 * D, device=dev)).to(dtype)
+        h2 = xs.to(dtype)
+        rec(f"kagolix {tag}/gemm {T}x{D}x{2 * D}", _timed(lambda: ops.matmul_nt(h2, wk), reps), 4.0 * T * D * D, es * (2 * D * D + 2 * T * D) + 4 * T * D)
+    return {"part": "kernels", "family": "nudadra", "dtype": str(dtype), "batch": B, "context": L, "kernels": res}
+
+
+# family -> (its stack, the closest existing stack beside it, its kernels one by one)
+FAMILIES = {
+    "lopilix": (lopilix_config, hybrid_config, bench_lopilix_kernels),
+    "gizezen": (gizezen_config, kagolix_attention_moe_config, bench_gizezen_kernels),
+    "sisavik": (sisavik_config, kagolix_dense_config, bench_sisavik_kernels),
+    "nudadra": (nudadra_config, kagolix_attention_mamba_config, bench_nudadra_kernels),
+}
+
+
 def main(a) -> int:
     """``bench.py --hybrid SIZE`` (one GPU)."""
     dev = torch.device("cuda", 0)
     torch.cuda.set_device(dev)
     z = SIZES[a.hybrid]
     dtype = torch.bfloat16 if a.hybrid_dtype == "bfloat16" else torch.float32
-    B, L = a.hybrid_batch, a.hybrid_context
+    B, L, steps = a.hybrid_batch, a.hybrid_context, a.steps * 8
     lines: List[dict] = []
-    parts = a.hybrid_parts.split(",")
-    if getattr(a, "hybrid_family", "kagolix") == "lopilix":
-        if "hybrid" in parts:
-            lines.append(bench_hybrid_model(z, dtype, B, L, a.steps * 8, dev, lopilix_config(z), "lopilix"))
+    fam = getattr(a, "hybrid_family", "kagolix")
+    if fam in FAMILIES:
+        own, other, kernels = FAMILIES[fam]
+        parts = {"hybrid": lambda: bench_hybrid_model(z, dtype, B, L, steps, dev, own(z), fam),
+                 "dense": lambda: bench_hybrid_model(z, dtype, B, L, steps, dev, other(z), "kagolix"),
+                 "kernels": lambda: kernels(z, dtype, B, L, dev)}
+    else:
+        parts = {"hybrid": lambda: bench_hybrid_model(z, dtype, B, L, steps, dev),
+                 "dense": lambda: bench_dense_model(z, 6, B, L, steps, dev),
+                 "kernels": lambda: bench_kernels(z, dtype, B, L, dev)}
+    for name, run in parts.items():
+        if name in a.hybrid_parts.split(","):
+            lines.append(run())
             print(json.dumps(lines[-1]), flush=True)
-        if "dense" in parts:      # (the closest existing model: the Kagolix stack of attention, recurrent and state-space layers)
-            lines.append(bench_hybrid_model(z, dtype, B, L, a.steps * 8, dev, hybrid_config(z), "kagolix"))
-            print(json.dumps(lines[-1]), flush=True)
-        if "kernels" in parts:
-            lines.append(bench_lopilix_kernels(z, dtype, B, L, dev))
-            print(json.dumps(lines[-1]), flush=True)
-        if a.json_out:
-            with open(a.json_out, "w") as f:
-                json.dump(lines, f, indent=1)
-        return 0
-    if getattr(a, "hybrid_family", "kagolix") == "gizezen":
-        if "hybrid" in parts:
-            lines.append(bench_hybrid_model(z, dtype, B, L, a.steps * 8, dev, gizezen_config(z), "gizezen"))
-            print(json.dumps(lines[-1]), flush=True)
-        if "dense" in parts:      # (the closest existing model: a Kagolix stack of attention layers with experts)
-            lines.append(bench_hybrid_model(z, dtype, B, L, a.steps * 8, dev, kagolix_attention_moe_config(z), "kagolix"))
-            print(json.dumps(lines[-1]), flush=True)
-        if "kernels" in parts:
-            lines.append(bench_gizezen_kernels(z, dtype, B, L, dev))
-            print(json.dumps(lines[-1]), flush=True)
-        if a.json_out:
-            with open(a.json_out, "w") as f:
-                json.dump(lines, f, indent=1)
-        return 0
-    if getattr(a, "hybrid_family", "kagolix") == "sisavik":
-        if "hybrid" in parts:
-            lines.append(bench_hybrid_model(z, dtype, B, L, a.steps * 8, dev, sisavik_config(z), "sisavik"))
-            print(json.dumps(lines[-1]), flush=True)
-        if "dense" in parts:      # (the closest existing model here: a Kagolix stack of equal width, depth and ff)
-            lines.append(bench_hybrid_model(z, dtype, B, L, a.steps * 8, dev, kagolix_dense_config(z), "kagolix"))
-            print(json.dumps(lines[-1]), flush=True)
-        if "kernels" in parts:
-            lines.append(bench_sisavik_kernels(z, dtype, B, L, dev))
-            print(json.dumps(lines[-1]), flush=True)
-        if a.json_out:
-            with open(a.json_out, "w") as f:
-                json.dump(lines, f, indent=1)
-        return 0
-    if "hybrid" in parts:
-        lines.append(bench_hybrid_model(z, dtype, B, L, a.steps * 8, dev))
-        print(json.dumps(lines[-1]), flush=True)
-    if "dense" in parts:
-        lines.append(bench_dense_model(z, 6, B, L, a.steps * 8, dev))
-        print(json.dumps(lines[-1]), flush=True)
-    if "kernels" in parts:
-        lines.append(bench_kernels(z, dtype, B, L, dev))
-        print(json.dumps(lines[-1]), flush=True)
     if a.json_out:
         with open(a.json_out, "w") as f:
             json.dump(lines, f, indent=1)

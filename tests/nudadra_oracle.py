@@ -107,7 +107,7 @@ def short_conv(u, w, b):
     """u: [T, C], w: [C, taps] (last column: the current row), zeros before the start."""
     T, taps = u.shape[0], w.shape[1]
     out = b[None].repeat(T, 1)
-    for back in range(taps):
+    for back in range(min(taps, T)):
         out[back:] += u[:T - back] * w[:, taps - 1 - back]
     return out
 

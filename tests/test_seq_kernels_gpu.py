@@ -696,3 +696,148 @@ def test_projected_rows_with_weighted_norms_before_the_rotation(ops, cdt, tol, H
         close(outs[0][0], outs[1][0], 3e-4)
         close(outs[0][1], outs[1][1], max(tol, 3e-4))
         close(outs[0][2], outs[1][2], tol)
+
+
+def blocks_of(lens, pos0, P, ps, dev, kcols, vcols, cdt, seed=3):
+    """Block pools in scattered pages: (block keys, block values, table, P), garbage where nothing is written."""
+    rng = np.random.default_rng(seed)
+    need = [max(1, -(-((p + n) // P) // ps)) for p, n in zip(pos0, lens)]
+    tab = np.full((len(lens), max(need)), -1, np.int32)
+    perm = rng.permutation(sum(need) + 3)
+    k = 0
+    for b, m in enumerate(need):
+        tab[b, :m] = perm[k:k + m]
+        k += m
+    pools = [torch.randn(sum(need) + 3, ps, c, device=dev).to(cdt) for c in (kcols, vcols)]
+    return pools[0], pools[1], torch.from_numpy(tab).to(dev), P
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+@pytest.mark.parametrize("P", [1, 3, 16, 40])
+@pytest.mark.parametrize("kcols,vcols", [(20, 14), (64, 128), (200, 36)])
+def test_block_means(ops, cdt, tol, P, kcols, vcols):
+    """Blocks completed by whole prompts, by portions that begin inside a block, and by single rows; rows of the
+    block pools that no completed block owns stay as they were."""
+    H, R = ops
+    torch.manual_seed(P + kcols)
+    for lens, pos0 in (([70, 5, 33], [0, 0, 0]), ([3, 40, 1], [70, 5, 33]), ([1, 1, 1], [39, 2, 15]), ([2, 2], [38, 0])):
+        md, npages, _ = meta_of(lens, pos0, DEV)
+        kc, vc = torch.randn(npages, 16, kcols, device=DEV).to(cdt), torch.randn(npages, 16, vcols, device=DEV).to(cdt)
+        b1 = blocks_of(lens, pos0, P, 16, DEV, kcols, vcols, cdt)
+        b2 = (b1[0].clone(), b1[1].clone()) + b1[2:]
+        H.block_means(kc, vc, b1, md, kcols, vcols)
+        R.block_means(kc, vc, b2, md, kcols, vcols)
+        for x, y in zip(b1[:2], b2[:2]):
+            close(x, y, 1e-6 if cdt == torch.float32 else 8e-3)
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+@pytest.mark.parametrize("Hh,G,d,dv,rot", [(6, 2, 10, 14, (6, 50.0, ("turns", 3.0, 24.0, 4.0, 0.5))), (8, 4, 64, 128, (64, 1e6, None)),
+                                           (4, 2, 128, 128, (128, 5e5, ("turns", 8.0, 128.0, 16.0, 1.0))), (2, 1, 96, 96, (96, 1e4, None)),
+                                           (2, 2, 150, 130, (140, 1e4, ("turns", 2.0, 64.0, 8.0, 1.0))), (3, 1, 300, 40, (20, 1e3, None)),
+                                           (3, 3, 8, 5, None)])
+def test_projected_rows_rotated_in_halves_with_block_means(ops, cdt, tol, Hh, G, d, dv, rot):
+    """One pass over projected rows with the half layout, amplified cosines and no norm, and the block means of the rows
+    it writes -- as a launch of its own for many rows, inside the same launch for one row each -- against the chain
+    of plain ops."""
+    H, R = ops
+    torch.manual_seed(d + dv)
+    for lens, pos0 in (([37, 1, 20], [0, 9, 130]), ([1, 1, 1, 1], [15, 4, 31, 200]), ([1, 1], [5, 11]), ([2], [10])):
+        md, npages, _ = meta_of(lens, pos0, DEV)
+        T = sum(lens)
+        z = torch.randn(T, (Hh + G) * d + G * dv + 5, device=DEV)
+        kc, vc = torch.randn(npages, 16, G * d, device=DEV).to(cdt), torch.randn(npages, 16, G * dv, device=DEV).to(cdt)
+        kc2, vc2 = kc.clone(), vc.clone()
+        q1, q2 = torch.empty(T, Hh * d, device=DEV), torch.empty(T, Hh * d, device=DEV)
+        b1 = blocks_of(lens, pos0, 6, 16, DEV, G * d, G * dv, cdt)
+        b2 = (b1[0].clone(), b1[1].clone()) + b1[2:]
+        kw = dict(rot=rot, norm=False, half=True)
+        H.qkv_conv_rope_store(z, None, None, md, Hh, G, d, dv, q1, kc, vc, blocks=b1, **kw)
+        R.qkv_conv_rope_store(z, None, None, md, Hh, G, d, dv, q2, kc2, vc2, blocks=b2, **kw)
+        close(q1, q2, 2e-5)
+        for x, y in ((kc, kc2), (vc, vc2), (b1[0], b2[0]), (b1[1], b2[1])):
+            close(x, y, tol)
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+@pytest.mark.parametrize("Hh,G,d,dv", [(6, 2, 10, 14), (3, 1, 64, 64), (4, 2, 96, 96), (4, 4, 32, 32), (4, 2, 128, 128), (2, 1, 64, 128),
+                                       (2, 2, 128, 64), (2, 1, 80, 48)])
+def test_attention_over_a_window_and_pooled_blocks(ops, cdt, tol, Hh, G, d, dv):
+    """Window tokens and earlier blocks in one softmax: prompts of several row tiles, portions, single rows, with head
+    gates; windows and blocks that divide a page, each other, or nothing; block pools wider than the heads need."""
+    H, R = ops
+    torch.manual_seed(d + dv)
+    for lens, pos0, window, P in (([300, 17, 140], [0, 0, 0], 50, 6), ([200, 30], [300, 17], 33, 16), ([3, 1, 1], [70, 5, 333], 9, 4),
+                                  ([260], [0], 1, 1), ([150, 20], [0, 40], 2, 40), ([1, 1], [600, 2], 70, 3), ([130], [0], 500, 8)):
+        md, npages, _ = meta_of(lens, pos0, DEV)
+        T = sum(lens)
+        kc, vc = torch.randn(npages, 16, G * d, device=DEV).to(cdt), torch.randn(npages, 16, G * dv, device=DEV).to(cdt)
+        kp, vp, tab, _ = blocks_of(lens, pos0, P, 16, DEV, G * d + 8, G * dv + 16, cdt)
+        q = torch.randn(T, Hh * d, device=DEV)
+        if cdt == torch.bfloat16:
+            q = q.to(cdt).float()
+        gate = torch.randn(T, Hh + 3, device=DEV)[:, 1:1 + Hh]
+        args = (q, kc, vc, md, Hh, G, d, dv, d ** -0.5 * 1.5, 0.0, None, None, 0, 16, cdt)
+        kw = dict(window=window, blocks=(kp, vp, tab, P), head_gate=gate)
+        close(H.attn_paged(*args, **kw), R.attn_paged(*args, **kw), tol)
+        o = torch.empty(T, Hh * dv, device=DEV)
+        close(H.attn_paged(*args, out=o, **kw), R.attn_paged(*args, **kw), tol)
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+def test_decode_rows_over_many_blocks_split_their_keys(ops, cdt, tol):
+    """Few rows over a long window and hundreds of blocks: the keys are cut into ranges whose first ones hold only
+    blocks; the merge applies the head gates."""
+    H, R = ops
+    torch.manual_seed(2)
+    Hh, G, d, dv, window, P = 4, 2, 40, 24, 700, 3
+    md, npages, _ = meta_of([1, 1], [3000, 900], DEV)
+    kc, vc = torch.randn(npages, 16, G * d, device=DEV).to(cdt), torch.randn(npages, 16, G * dv, device=DEV).to(cdt)
+    blocks = blocks_of([1, 1], [3000, 900], P, 16, DEV, G * d, G * dv, cdt)
+    q, gate = torch.randn(2, Hh * d, device=DEV), torch.randn(2, Hh, device=DEV)
+    args = (q, kc, vc, md, Hh, G, d, dv, 0.3, 0.0, None, None, 0, 16, cdt)
+    kw = dict(window=window, blocks=blocks, head_gate=gate)
+    close(H.attn_paged(*args, **kw), R.attn_paged(*args, **kw), tol)
+    with pytest.raises(ValueError):
+        H.attn_paged(*args, window=0, blocks=blocks)
+    with pytest.raises(ValueError):
+        H.attn_paged(*args, window=window, sink=0.0, blocks=blocks)
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+@pytest.mark.parametrize("D", [1, 35, 96, 2048, 2300, 4096, 8200, 8196])
+def test_residual_update_from_two_normed_branches(ops, cdt, tol, D):
+    """All parts together and each left out; rows that are column blocks of a wider buffer (whose other columns stay);
+    widths that fit the registers and wider ones; one-number and vector weights of the norm behind it."""
+    H, R = ops
+    torch.manual_seed(D)
+    T = 7
+    wide = torch.randn(T, 2 * D, device=DEV)
+    a, b, f = (torch.randn(T, D, device=DEV) * s for s in (3.0, 0.2, 1.0))
+    wa, wb, nw = (torch.randn(D, device=DEV) for _ in range(3))
+    one = torch.tensor([0.7], device=DEV)
+    for kw in (dict(branches=((a, wa), (b, wb)), coef=0.5, add=f), dict(branches=((a, wa), (b, wb)), coef=1.3),
+               dict(branches=((a, wa), (b, wb)), coef=0.5, add=f, norm_w=nw), dict(add=f, keep=False, norm_w=one),
+               dict(add=f, keep=False), dict(add=f, norm_w=one), dict(norm_w=nw)):
+        x1, x2 = wide.clone(), wide.clone()
+        h1 = H.residual_branches_(x1[:, :D], eps=1e-6, out_dtype=cdt, **kw)
+        h2 = R.residual_branches_(x2[:, :D], eps=1e-6, out_dtype=cdt, **kw)
+        close(x1, x2, 1e-5)
+        assert torch.equal(x1[:, D:], wide[:, D:])
+        if "norm_w" in kw:
+            close(h1, h2, tol)
+        else:
+            assert h1 is None and h2 is None
+    idx = torch.tensor([6, 0, 3], dtype=torch.int32, device=DEV)
+    close(H.group_rmsnorm(wide[:, :D], one, 1, 1e-6, cdt, row_idx=idx), R.group_rmsnorm(wide[:, :D], one, 1, 1e-6, cdt, row_idx=idx), tol)
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+@pytest.mark.parametrize("M,N,K", [(5, 70, 33), (130, 192, 256), (300, 200, 454), (1600, 4200, 136), (8, 200, 512), (1, 33, 72)])
+def test_squared_relu_in_the_epilogue(ops, cdt, tol, M, N, K):
+    H, R = ops
+    torch.manual_seed(M + N)
+    a, w = torch.randn(M, K, device=DEV).to(cdt), torch.randn(N, K, device=DEV).to(cdt)
+    b = torch.randn(N, device=DEV)
+    close(H.matmul_nt(a, w, relu2=True, out_dtype=cdt), R.matmul_nt(a, w, relu2=True, out_dtype=cdt), tol)
+    close(H.matmul_nt(a, w, b, relu2=True), R.matmul_nt(a, w, b, relu2=True), 2e-5)
