@@ -45,7 +45,7 @@ int fls_seq_gather_rows(const void* x, int tx, int ldx, const int* idx, void* y,
 int fls_seq_xielu(const float* z, int ldz, const float* act, void* y, int ty, int ldy, int rows, int cols, fls_stream_t s);
 // y[r, c] = act(gu[r, c]) * gu[r, cols + c]; act: 0 = silu, 1 = gelu (tanh form)
 int fls_seq_gate_mul(const float* gu, int ldg, void* y, int ty, int ldy, int rows, int cols, int act, fls_stream_t s);
-// y = f(z) elementwise; kind: 0 = tanh, 1 = gelu (exact: 0.5 z (1 + erf(z / sqrt 2)))
+// y = f(z) elementwise; kind: 0 = tanh, 1 = gelu (exact: 0.5 z (1 + erf(z / sqrt 2))), 2 = z (a cast)
 int fls_seq_unary(const float* z, int ldz, void* y, int ty, int ldy, int rows, int cols, int kind, fls_stream_t s);
 // per row t and head h: the n entries x[t, x_col + h x_hs ...] (x of type tx), RMS-normed over n times w[n] (w != null), the first
 // rot entries rotated in pairs (2i, 2i+1) by the angle tok_pos[t] * freqs[i]; written as type to at

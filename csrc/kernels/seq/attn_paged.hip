@@ -82,7 +82,9 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
   const int nkeep = POOL ? (i - window + 1 > 0 ? (i - window + 1) / ab.P : 0) : min(keep_first, lo);
   const int* btable = POOL ? ab.table + (size_t)tok_seq[t] * ab.t_stride : nullptr;
   const int nkeys = nkeep + i - lo + 1;
-  const int ntiles = (nkeys + 63) / 64;
+  // (with blocks every tile holds keys of one kind: nbt tiles of blocks, then tiles of tokens)
+  const int nbt = POOL ? (nkeep + 63) / 64 : 0;
+  const int ntiles = POOL ? nbt + (i - lo) / 64 + 1 : (nkeys + 63) / 64;
   const float a1 = r1 != nullptr ? r1[h] : 0.f, a2 = r2 != nullptr ? r2[h] : 0.f;
   const bool gated = gate_bias != nullptr;
   const float gb = gated ? gate_bias[h] : 0.f;
@@ -96,20 +98,20 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
   const int tps = (ntiles + nsplit - 1) / nsplit;
   const int tile_hi = min(ntiles, ((int)blockIdx.z + 1) * tps);
   for (int tile = blockIdx.z * tps + wave; tile < tile_hi; tile += 4) {
-    const int n = tile * 64 + lane;
-    const bool valid = n < nkeys;
-    const int j = n < nkeep ? n : lo + (n - nkeep);
+    const bool pooled = POOL && tile < nbt;        // (wave-uniform)
+    const int n = POOL ? (pooled ? tile : tile - nbt) * 64 + lane : tile * 64 + lane;
+    const int tkeys = POOL ? (pooled ? nkeep : i - lo + 1) : nkeys;
+    const bool valid = n < tkeys;
+    const int j = POOL ? (pooled ? n : lo + n) : (n < nkeep ? n : lo + (n - nkeep));
+    const int* tab = pooled ? btable : table;
+    const T* kb = pooled ? reinterpret_cast<const T*>(ab.kp) : kc;
+    const T* vb = (pooled ? reinterpret_cast<const T*>(ab.vp) : vc) + (size_t)gv * dv;
+    const int lk = pooled ? ab.ldk : ldk, lv = pooled ? ab.ldv : ldv;
     float sc = -1e30f;
     int row = 0;
     if (valid) {
-      if (POOL && n < nkeep) {
-        row = btable[n / page_size] * page_size + n % page_size;
-        sc = dot_row<T>(reinterpret_cast<const T*>(ab.kp) + (size_t)row * ab.ldk + (size_t)g * d, qs, d, vec) * scale;
-        row = ~row;                                // (a row of the block pools)
-      } else {
-        row = table[j / page_size] * page_size + j % page_size;
-        sc = dot_row<T>(kc + (size_t)row * ldk + (size_t)g * d, qs, d, vec) * scale;
-      }
+      row = tab[j / page_size] * page_size + j % page_size;
+      sc = dot_row<T>(kb + (size_t)row * lk + (size_t)g * d, qs, d, vec) * scale;
       if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
       if (a1 != 0.f) sc -= a1 * log1pf(a2 * (float)(i - j));
     }
@@ -129,11 +131,7 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
     // but the compiler must not move the loads above the stores)
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
-    const int nk = min(64, nkeys - tile * 64);
-    auto vrow = [&](int r) -> const T* {
-      if (POOL && r < 0) return reinterpret_cast<const T*>(ab.vp) + (size_t)(~r) * ab.ldv + (size_t)gv * dv;
-      return vc + (size_t)r * ldv + (size_t)gv * dv;
-    };
+    const int nk = min(64, tkeys - (n - lane));
 #pragma unroll
     for (int c = 0; c < MAX_DV_PER_LANE; ++c) {
       const int e = lane + 64 * c;
@@ -143,11 +141,11 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
         for (; jj + 8 <= nk; jj += 8) {            // eight independent value loads in flight
           float v[8];
 #pragma unroll
-          for (int x = 0; x < 8; ++x) v[x] = ldf(vrow(prow[wave][jj + x]), e);
+          for (int x = 0; x < 8; ++x) v[x] = ldf(vb + (size_t)prow[wave][jj + x] * lv, e);
 #pragma unroll
           for (int x = 0; x < 8; ++x) a += pw[wave][jj + x] * v[x];
         }
-        for (; jj < nk; ++jj) a += pw[wave][jj] * ldf(vrow(prow[wave][jj]), e);
+        for (; jj < nk; ++jj) a += pw[wave][jj] * ldf(vb + (size_t)prow[wave][jj] * lv, e);
         acc[c] = a;
       }
     }

@@ -31,8 +31,9 @@ typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 #define KT 32             // keys per tile
 #define PLD (KT + 8)      // row stride (elements) of the transposed V tile and of the weight tiles
 
+// (two waves per SIMD: a few registers over 256 would halve that)
 template <int D, int DV, typename TQ, typename TO, bool POOL>
-__global__ __launch_bounds__(256) void attn_prefill_kernel(const TQ* __restrict__ q, int ldq, const bf16_t* __restrict__ kc, int ldk,
+__global__ __launch_bounds__(256, 2) void attn_prefill_kernel(const TQ* __restrict__ q, int ldq, const bf16_t* __restrict__ kc, int ldk,
                                                            const bf16_t* __restrict__ vc, int ldv, TO* __restrict__ out, int ldo,
                                                            const int* __restrict__ tiles, const int* __restrict__ tok_seq,
                                                            const int* __restrict__ tok_pos, const int* __restrict__ page_table,

@@ -235,7 +235,7 @@ extern "C" int fls_seq_gate_mul(const float* gu, int ldg, void* y, int ty, int l
   return 0;
 }
 
-// y = f(z) elementwise; kind: 0 = tanh, 1 = gelu in its exact form 0.5 z (1 + erf(z / sqrt 2))
+// y = f(z) elementwise; kind: 0 = tanh, 1 = gelu in its exact form 0.5 z (1 + erf(z / sqrt 2)), 2 = z itself (a cast)
 template <typename TO>
 __global__ void unary_kernel(const float* __restrict__ z, int ldz, TO* __restrict__ y, int ldy, int cols, int kind) {
   const float* zr = z + (size_t)blockIdx.x * ldz;
@@ -247,9 +247,36 @@ __global__ void unary_kernel(const float* __restrict__ z, int ldz, TO* __restric
   for (int c = threadIdx.x; c < cols; c += blockDim.x) stf(yr, c, tanhf(zr[c]));
 }
 
+template <typename TO>
+__global__ __launch_bounds__(256) void cast_kernel(const float* __restrict__ z, int ldz, TO* __restrict__ y, int ldy, int cols, int vec) {
+  const float* zr = z + (size_t)blockIdx.x * ldz;
+  TO* yr = y + (size_t)blockIdx.x * ldy;
+  const int c0 = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (c0 >= cols) return;
+  if (vec) {
+    const float4 v = *reinterpret_cast<const float4*>(zr + c0);
+    if constexpr (sizeof(TO) == 2) {
+      const bf16_t e[4] = {f_to_bf16(v.x), f_to_bf16(v.y), f_to_bf16(v.z), f_to_bf16(v.w)};
+      *reinterpret_cast<uint2*>(yr + c0) = *reinterpret_cast<const uint2*>(e);
+    } else {
+      *reinterpret_cast<float4*>(yr + c0) = v;
+    }
+  } else {
+    for (int c = c0; c < min(cols, c0 + 4); ++c) stf(yr, c, zr[c]);
+  }
+}
+
 extern "C" int fls_seq_unary(const float* z, int ldz, void* y, int ty, int ldy, int rows, int cols, int kind, fls_stream_t s) {
   if (rows <= 0) return 0;
-  if (kind != 0 && kind != 1) return -1;
+  if (kind < 0 || kind > 2) return -1;
+  if (kind == 2) {
+    const int vec = cols % 4 == 0 && ldz % 4 == 0 && ldy % 4 == 0 && (uintptr_t)z % 16 == 0 && (uintptr_t)y % 16 == 0;
+    dim3 grid(rows, (cols + 1023) / 1024);
+    if (ty == 1) hipLaunchKernelGGL((cast_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)s, z, ldz, (bf16_t*)y, ldy, cols, vec);
+    else hipLaunchKernelGGL((cast_kernel<float>), grid, dim3(256), 0, (hipStream_t)s, z, ldz, (float*)y, ldy, cols, vec);
+    SEQ_LAUNCH_CHECK();
+    return 0;
+  }
   if (ty == 1) hipLaunchKernelGGL((unary_kernel<bf16_t>), dim3(rows), dim3(256), 0, (hipStream_t)s, z, ldz, (bf16_t*)y, ldy, cols, kind);
   else hipLaunchKernelGGL((unary_kernel<float>), dim3(rows), dim3(256), 0, (hipStream_t)s, z, ldz, (float*)y, ldy, cols, kind);
   SEQ_LAUNCH_CHECK();

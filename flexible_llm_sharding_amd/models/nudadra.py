@@ -151,8 +151,8 @@ def run_block(ctx, W, xs: torch.Tensor, meta: dict, name: str) -> torch.Tensor:
     if t is None:
         h = ops.group_rmsnorm(x, W["norm1"], 1, eps, out_dtype=cdt)
     else:                                                                   # the row is replaced: W_in [x; x0] + step_t
-        h = ops.residual_branches_(x, add=ops.matmul_nt(xs, W["loop_in"], bias=W["loop_step"][t]), keep=False, eps=eps,
-                                   norm_w=W["norm1"], out_dtype=cdt)
+        entry = ops.matmul_nt(ops.cast_rows(xs, cdt), W["loop_in"], bias=W["loop_step"][t])
+        h = ops.residual_branches_(x, add=entry, keep=False, eps=eps, norm_w=W["norm1"], out_dtype=cdt)
     c = _cols(L.mixer)
     z = ops.matmul_nt(h, W["win"])                                          # fp32 [T, q | k | v | z | xBC | dt | g]
     left = _attention(ctx, L.mixer["left"], W, z, c, meta, name)

@@ -442,6 +442,15 @@ class HipSeqOps:
     def silu_mul(self, gu, out_dtype):
         return self.gate_mul(gu, out_dtype, "silu")
 
+    def cast_rows(self, z, out_dtype):
+        _rows(z, "z", torch.float32)
+        if out_dtype == torch.float32:
+            return z
+        y = torch.empty(z.shape, dtype=out_dtype, device=z.device)
+        _chk(self.k.fls_seq_unary(z.data_ptr(), z.stride(0), y.data_ptr(), _CODE[out_dtype], z.shape[1], z.shape[0], z.shape[1], 2,
+                                  _stream()), "fls_seq_unary")
+        return y
+
     def unary(self, z, kind, out_dtype):
         _rows(z, "z", torch.float32)
         if kind not in ("tanh", "gelu"):
@@ -621,7 +630,7 @@ class HipSeqOps:
                 _chk(rc, "fls_seq_attn_heads")
         # few rows over many keys (decoding a small batch): cut every row's keys into ranges that run as
         # blocks of their own, so that the launch has a few hundred blocks
-        nsplit = max(1, min(8, 512 // max(1, T * H), bound // 256))
+        nsplit = max(1, min(8, 512 // max(1, T * H), bound // 256 if blocks is None else -(-bound // 256)))
         part = torch.empty(T * H * nsplit * (dv + 4), dtype=torch.float32, device=q.device) if nsplit > 1 else None
         _chk(self.k.fls_seq_attn_paged(q.data_ptr(), q.stride(0), _code(q, "q"), kcache.data_ptr(), ldk, vcache.data_ptr(), ldv,
                                        _code(kcache, "kcache"), out.data_ptr(), to, out.stride(0), meta["tok_seq"].data_ptr(),

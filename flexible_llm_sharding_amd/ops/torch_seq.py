@@ -170,6 +170,10 @@ class TorchSeqOps:
     def silu_mul(self, gu, out_dtype):
         return self.gate_mul(gu, out_dtype, "silu")
 
+    def cast_rows(self, z, out_dtype):
+        """fp32 rows as the next product's operand (fp32: the rows themselves)."""
+        return z.to(out_dtype)
+
     def unary(self, z, kind, out_dtype):
         """tanh, or gelu: the exact form 0.5 z (1 + erf(z / sqrt 2))."""
         if kind == "gelu":

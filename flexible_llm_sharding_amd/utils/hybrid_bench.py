@@ -840,8 +840,8 @@ def bench_nudadra_kernels(z: dict, dtype, B: int, L: int, dev) -> dict:
             es * (fw * D + T * D + T * fw))
         wl = (0.02 * torch.randn(D, 2 * D, device=dev)).to(dtype)
         xs, sv = torch.randn(T, 2 * D, device=dev), torch.randn(D, device=dev)
-        rec(f"{tag}/pass entry gemm {T}x{D}x{2 * D}, fp32 rows", _timed(lambda: ops.matmul_nt(xs, wl, bias=sv), reps), 4.0 * T * D * D,
-            es * 2 * D * D + 12 * T * D)
+        rec(f"{tag}/pass entry: cast + gemm {T}x{D}x{2 * D}", _timed(lambda: ops.matmul_nt(ops.cast_rows(xs, dtype), wl, bias=sv), reps),
+            4.0 * T * D * D, es * 2 * D * D + T * D * (8 + 4 * es + 4))
         wk = (0.02 * torch.randn(D, 2 * D, device=dev)).to(dtype)
         h2 = xs.to(dtype)
         rec(f"kagolix {tag}/gemm {T}x{D}x{2 * D}", _timed(lambda: ops.matmul_nt(h2, wk), reps), 4.0 * T * D * D, es * (2 * D * D + 2 * T * D) + 4 * T * D)

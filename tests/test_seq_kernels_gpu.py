@@ -841,3 +841,7 @@ def test_squared_relu_in_the_epilogue(ops, cdt, tol, M, N, K):
     b = torch.randn(N, device=DEV)
     close(H.matmul_nt(a, w, relu2=True, out_dtype=cdt), R.matmul_nt(a, w, relu2=True, out_dtype=cdt), tol)
     close(H.matmul_nt(a, w, b, relu2=True), R.matmul_nt(a, w, b, relu2=True), 2e-5)
+    z = torch.randn(M, K + 3, device=DEV)[:, 1:1 + K]
+    assert torch.equal(H.cast_rows(z, cdt), R.cast_rows(z, cdt)) and H.cast_rows(z, cdt).dtype == cdt
+    z = torch.randn(M, 4 * K, device=DEV)
+    assert torch.equal(H.cast_rows(z, cdt), z.to(cdt))
