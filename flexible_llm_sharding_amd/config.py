@@ -966,9 +966,139 @@ class NudadraConfig:
         return d
 
 
+NUMOLORN_MIXERS = ("latent_attention", "latent_attention_2", "channel_delta")
+
+
+@dataclass
+class NumolornConfig:
+    """Numolorn: a decoder whose layers run a mixer and a feed-forward side by side, each on a norm of its own of the
+    same row and scaled per channel, x <- x + (mixer(N1(x)) ls1 + ff(N2(x)) ls2).  The embedding row is the token's plus
+    a hashed bigram's (the token and the one before it).  Mixers: latent attention (queries through a latent,
+    keys and values made from one cached latent row and a rotated key part shared by all heads, a learned softmax
+    sink and a sigmoid gate per head), latent attention without positions over a sliding window, and a gated delta
+    rule with one decay per head and key channel.  Feed-forwards: SiLU-gated dense, or a mixture of clamped experts
+    and identity experts chosen by corrected softmax scores among the best groups.  ``loop``: layers start .. stop - 1
+    run ``times`` times in a row on the same weights; every pass but the first adds the embedding row, and every pass
+    has a state of its own (its layers are names of their own, ``l0@1``).  Everything is read from config.json:
+    ``width``, ``vocab``, ``norm.eps``, ``logit_scale``, ``embedding.bigram``, ``loop`` and ``layers`` (per layer
+    ``type``, ``mixer``, ``mlp``); the ranks of the delta rule's two-layer maps, which it leaves open, come from the
+    checkpoint's tensor shapes."""
+    width: int
+    vocab: int
+    norm_eps: float
+    logit_scale: float
+    bigram: Optional[dict]
+    loop: Optional[dict]
+    layers: list
+    family = "numolorn"
+    model_type = "numolorn"
+    is_moe = False
+    sliding_window = None
+    tie_word_embeddings = True
+
+    hidden_size = KagolixConfig.hidden_size
+    vocab_size = KagolixConfig.vocab_size
+    save = KagolixConfig.save
+    order = LopilixConfig.order
+    num_hidden_layers = LopilixConfig.num_hidden_layers
+    num_layers_total = LopilixConfig.num_layers_total
+    layer_names = LopilixConfig.layer_names
+    layer = LopilixConfig.layer
+    total_params = LopilixConfig.total_params
+
+    @property
+    def loops(self) -> bool:
+        """Whether some layers run more than once."""
+        return bool(self.loop) and int(self.loop["times"]) > 1 and int(self.loop["start"]) < int(self.loop["stop"])
+
+    @property
+    def state_width(self) -> int:
+        """Columns of the activation that passes from layer to layer: the residual row, and beside it the embedding
+        row when later passes of a loop add it."""
+        return (2 if self.loops else 1) * self.width
+
+    def reenters(self, name: str) -> bool:
+        """Whether layer run ``name`` opens a pass other than the first (the embedding row joins the residual row)."""
+        i, _, p = name[1:].partition("@")
+        return self.loops and int(p or 0) > 0 and int(i) == int(self.loop["start"])
+
+    def validate(self) -> None:
+        lp = self.loop
+        if lp and not (0 <= int(lp["start"]) <= int(lp["stop"]) <= len(self.layers) and int(lp["times"]) >= 1):
+            raise ValueError(f"loop {lp} does not fit {len(self.layers)} layers")
+        if self.bigram is not None and int(self.bigram["buckets"]) < 1:
+            raise ValueError(f"embedding.bigram {self.bigram}")
+        for i, l in enumerate(self.layers):
+            m = l.mixer
+            if l.type not in NUMOLORN_MIXERS:
+                raise NotImplementedError(f"layer {i}: mixer type {l.type!r}")
+            if l.type == "channel_delta":
+                if m["heads"] % m["kv_heads"]:
+                    raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+                if int(m["conv"]) < 1:
+                    raise ValueError(f"layer {i}: conv must be >= 1 taps")
+                if not 1 <= int(m["dim"]) <= 256 or int(m["vdim"]) > 512:
+                    # (the scan keeps a value column's key rows in the registers of 16 lanes, up to 16 rows each)
+                    raise NotImplementedError(f"layer {i}: a recurrent state of {m['dim']} x {m['vdim']} per head")
+            else:
+                dr = int(m["rot_dim"]) if l.type == "latent_attention" else 0
+                if dr and (int(m["rot"]["dims"]) > dr or int(m["rot"]["dims"]) % 2):
+                    raise ValueError(f"layer {i}: rot.dims must be even and at most rot_dim")
+                if int(m["kv_rank"]) > 512 or int(m["kv_rank"]) + dr > 1024 or max(int(m["dim"]), int(m["vdim"]), dr) > 512:
+                    # (the paged attention kernel of csrc/kernels/seq: a latent row is its key and its value)
+                    raise NotImplementedError(f"layer {i}: latent rows above 512 + 512 or head sizes above 512")
+                if m.get("mask") is not None and int(m["mask"]["size"]) < 1:
+                    raise ValueError(f"layer {i}: mask {m['mask']}")
+            if l.mlp is None:
+                continue
+            if l.mlp["kind"] not in ("dense", "moe"):
+                raise NotImplementedError(f"layer {i}: mlp kind {l.mlp['kind']!r}")
+            if l.mlp["kind"] == "moe":
+                r = l.mlp["router"]
+                E = int(r["experts"]) + int(r.get("identity", 0))
+                if not 1 <= int(r["top"]) <= min(E, 16) or E > 1024 or int(r["experts"]) < 1:
+                    raise NotImplementedError(f"layer {i}: router {r}")
+                g = r.get("groups")
+                if g and int(g["count"]) > 64:
+                    raise NotImplementedError(f"layer {i}: more than 64 expert groups")
+                if g and (E % int(g["count"]) or not 1 <= int(g["keep"]) <= int(g["count"])
+                          or int(g["keep"]) * (E // int(g["count"])) < int(r["top"])):
+                    raise ValueError(f"layer {i}: router groups {g} do not fit {E} experts, top {r['top']}")
+
+    @classmethod
+    def from_dict(cls, d: dict, model_path: Optional[str] = None) -> "NumolornConfig":
+        layers = [HybridLayer(l["type"], json.loads(json.dumps(l["mixer"])),
+                              None if l.get("mlp") is None else json.loads(json.dumps(l["mlp"]))) for l in d["layers"]]
+        shapes = None
+        for i, l in enumerate(layers):
+            for key, tensor in (("decay_rank", "a1"), ("gate_rank", "g1")) if l.type == "channel_delta" else ():
+                if key in l.mixer:
+                    continue
+                if shapes is None:
+                    if model_path is None:
+                        raise ValueError(f"layer {i}: {key} is neither given nor readable from a checkpoint")
+                    from .utils.safetensors_io import read_header
+                    shapes = {k: tuple(v.shape) for k, v in read_header(os.path.join(model_path, "model.safetensors"))[0].items()}
+                l.mixer[key] = int(shapes[f"l{i}.mix.{tensor}"][0])
+        cfg = cls(int(d["width"]), int(d["vocab"]), float(d["norm"]["eps"]), float(d.get("logit_scale", 1.0)),
+                  json.loads(json.dumps((d.get("embedding") or {}).get("bigram"))), json.loads(json.dumps(d.get("loop"))) or None, layers)
+        cfg.validate()
+        return cfg
+
+    def to_dict(self) -> dict:
+        d = {"architecture": "Numolorn", "width": self.width, "vocab": self.vocab, "norm": {"eps": self.norm_eps},
+             "logit_scale": self.logit_scale, "embedding": {},
+             "layers": [{"type": l.type, "mixer": l.mixer, "mlp": l.mlp} for l in self.layers]}
+        if self.bigram is not None:
+            d["embedding"]["bigram"] = self.bigram
+        if self.loop:
+            d["loop"] = self.loop
+        return d
+
+
 # "architecture" of config.json -> config class of a stateful hybrid family
 ARCHITECTURES = {"Kagolix": KagolixConfig, "Sisavik": SisavikConfig, "Gizezen": GizezenConfig, "Lopilix": LopilixConfig,
-                 "Nudadra": NudadraConfig}
+                 "Nudadra": NudadraConfig, "Numolorn": NumolornConfig}
 
 
 def load_config(model_path: str):
@@ -980,7 +1110,7 @@ def load_config(model_path: str):
     if arch is not None:
         if arch not in ARCHITECTURES:
             raise NotImplementedError(f"architecture {arch!r}: supported are {sorted(ARCHITECTURES)}")
-        if arch in ("Sisavik", "Lopilix"):             # (they read what config.json leaves open from the checkpoint's header)
+        if arch in ("Sisavik", "Lopilix", "Numolorn"):             # (they read what config.json leaves open from the checkpoint's header)
             return ARCHITECTURES[arch].from_dict(d, model_path)
         return ARCHITECTURES[arch].from_dict(d)
     return ModelConfig.from_dict(d)

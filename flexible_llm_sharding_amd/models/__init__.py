@@ -20,4 +20,7 @@ def hybrid_family(cfg):
     if fam == "nudadra":
         from . import nudadra
         return nudadra
+    if fam == "numolorn":
+        from . import numolorn
+        return numolorn
     raise NotImplementedError(f"no hybrid family {fam!r}")

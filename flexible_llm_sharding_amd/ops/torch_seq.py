@@ -28,12 +28,19 @@ class SeqRoute:
 
 class TorchSeqOps:
     # ----------------------------------------------------------------- rows
-    def embed_rows(self, ids, table, out=None, scale=1.0, pos_table=None, tok_pos=None, copies=1):
+    def embed_rows(self, ids, table, out=None, scale=1.0, pos_table=None, tok_pos=None, copies=1, bigram=None):
         """out[t] = table[ids[t]] * scale (+ pos_table[tok_pos[t]], a learned position vector), written
-        ``copies`` times side by side (the start of that many residual streams)."""
+        ``copies`` times side by side (the start of that many residual streams).  ``bigram`` = (table [buckets + 1, D], the
+        token before each, mul_prev, mul_cur): plus row (prev * mul_prev + id * mul_cur) mod buckets of that table, its last row
+        where nothing comes before (prev < 0)."""
         e = table.index_select(0, ids.long()).float()
         if scale != 1.0:
             e = e * scale
+        if bigram is not None:
+            bt, prev, mp, mc = bigram
+            n, prev = bt.shape[0] - 1, prev.long()
+            row = torch.where(prev < 0, torch.full_like(prev, n), (prev * int(mp) + ids.long() * int(mc)) % n)
+            e = e + bt.index_select(0, row).float()
         if pos_table is not None:
             e = e + pos_table.index_select(0, tok_pos.long()).float()
         if copies > 1:
@@ -69,6 +76,30 @@ class TorchSeqOps:
             new += add.float()
         x.copy_(new)
         return None if norm_w is None else self.group_rmsnorm(x, norm_w, 1, eps, out_dtype)
+
+    def rmsnorm_pair(self, x, w1, w2, eps, out_dtype, add=None):
+        """Two norms of one row that share its statistics: (rms(x) * w1, rms(x) * w2), the second None without ``w2``.
+        ``add``: first x += add, in the same pass."""
+        if add is not None:
+            x.add_(add.float())
+        h1 = self.group_rmsnorm(x, w1, 1, eps, out_dtype)
+        return h1, None if w2 is None else self.group_rmsnorm(x, w2, 1, eps, out_dtype)
+
+    def parallel_update_(self, x, a, wa, b=None, wb=None, moe=None):
+        """x += a * wa + f * wb, two sublayers of one row scaled per channel; f is ``b``, or with ``moe`` = (y, route, h, E)
+        the chosen experts' weighted sum: sum_k w[t, k] (y[dest[t, k]] if ids[t, k] < E else h[t]) (router outputs from E on
+        are identity experts), or nothing (``wb`` None)."""
+        new = a.float() * wa.float()
+        if moe is not None:
+            y, route, h, E = moe
+            T, top = route.dest.shape
+            ye = y.index_select(0, route.dest.long().reshape(-1)).reshape(T, top, -1)
+            rows = torch.where((route.ids < E)[:, :, None], ye.float(), h.float()[:, None, :])
+            b = (rows * route.w[:, :, None]).sum(1)
+        if b is not None:
+            new = new + b.float() * wb.float()
+        x.add_(new)
+        return x
 
     def dyt_norm(self, x, wb, alpha, out_dtype, row_idx=None):
         """Dynamic Tanh: tanh(alpha x) w + b elementwise, no statistics of the row; ``wb`` = [w; b] ([2, D]),
@@ -155,10 +186,14 @@ class TorchSeqOps:
         neg = an * (torch.expm1(torch.clamp(z, max=0.0)) - z) + 0.5 * z
         return torch.where(z > 0, pos, neg).to(out_dtype)
 
-    def gate_mul(self, gu, out_dtype, act="silu"):
-        """act(gu[:, :ff]) * gu[:, ff:]; act: silu or gelu_tanh."""
+    def gate_mul(self, gu, out_dtype, act="silu", limit=0.0, alpha=1.702):
+        """act(gu[:, :ff]) * gu[:, ff:]; act: silu or gelu_tanh; "clamped": g = min(gate, limit), u = up clamped to
+        +- limit, g sigmoid(alpha g) (u + 1)."""
         ff = gu.shape[1] // 2
         g, u = gu[:, :ff].float(), gu[:, ff:].float()
+        if act == "clamped":
+            g, u = g.clamp(max=float(limit)), u.clamp(-float(limit), float(limit))
+            return (g * torch.sigmoid(alpha * g) * (u + 1)).to(out_dtype)
         if act == "silu":
             a = g * torch.sigmoid(g)
         elif act == "gelu_tanh":
@@ -268,6 +303,16 @@ class TorchSeqOps:
                 raw[rows, out_col + h * out_hs:out_col + h * out_hs + n] = keep[:, h].to(raw.dtype)
         return out
 
+    def latent_rows(self, z, q_rank, r, dr, q_norm, kv_norm, eps, rot, rows, meta, out_dtype):
+        """The projected rows z = [query latent (q_rank) | latent (r) | rotated key part (dr) | ...] of a latent attention in
+        one pass: the query latent RMS-normed times ``q_norm`` (returned as ``out_dtype``; None without one), the latent normed
+        times ``kv_norm`` and the key part rotated in pairs (i, i + dims / 2) into row ``kv_slot[t]`` of the pool ``rows``
+        ([.., r + dr])."""
+        self.head_norm_rope(z, 1, r, q_rank, 0, rows, 0, 0, meta, w=kv_norm, eps=eps, row_map=meta["kv_slot"])
+        if dr:
+            self.head_norm_rope(z, 1, dr, q_rank + r, 0, rows, r, 0, meta, rot=rot, row_map=meta["kv_slot"], half=True)
+        return self.group_rmsnorm(z[:, :q_rank], q_norm, 1, eps, out_dtype) if q_rank else None
+
     def block_means(self, kc, vc, blocks, meta, kcols, vcols):
         """``blocks`` = (block keys, block values, table, P): every block of P positions (b P .. b P + P - 1) that this
         step's rows complete gets its mean key and mean value, over the rows as the pools hold them, written to row b of the
@@ -335,8 +380,8 @@ class TorchSeqOps:
         ``keep_first`` keys of the sequence), read from the request's pages.  Head h of H reads key /
         value head h // (H / G): the first G * d (G * dv) columns of a pool row.  Weights: softmax over
         the visible keys of cap(scale q.k) - r1 log(1 + r2 (i - j)), or, with ``gate_bias`` [H],
-        sigmoid(scale q.k + gate_bias[h]) for each key by itself.  ``sink`` (a number): the softmax has one
-        more entry of that score and no value, p_j = exp(s_j) / (exp(sink) + sum exp(s)).  ``head_gate``
+        sigmoid(scale q.k + gate_bias[h]) for each key by itself.  ``sink`` (a number, or one per head, fp32 [H]): the softmax has
+        one more entry of that score and no value, p_j = exp(s_j) / (exp(sink) + sum exp(s)).  ``head_gate``
         [T, H] fp32: head h's output of row t times sigmoid(head_gate[t, h]).  The result times ``out_scale``.
         ``v_heads`` (a divisor of G): the pool holds only that many value heads, key head g reads value
         head g % v_heads (several score maps over the same values).  ``out`` may be fp32 over bf16 pools.
@@ -377,7 +422,8 @@ class TorchSeqOps:
             if gate_bias is not None:
                 p = torch.sigmoid(s + gate_bias.float()[:, None])
             elif sink is not None:
-                p = torch.softmax(torch.cat([s, torch.full((H, 1), float(sink), device=q.device)], -1), -1)[:, :-1]
+                si = sink.float()[:, None] if torch.is_tensor(sink) else torch.full((H, 1), float(sink), device=q.device)
+                p = torch.softmax(torch.cat([s, si], -1), -1)[:, :-1]
             else:
                 p = torch.softmax(s, -1)
             o = torch.einsum("hn,nhv->hv", p, vv.repeat_interleave(rep, 1))
@@ -438,6 +484,34 @@ class TorchSeqOps:
         y = o.reshape(T, H * d) * norm_w.float() * torch.sigmoid(g.float()) * out_scale
         out.copy_(y.to(out.dtype))
         return out
+
+    def gated_delta_scan(self, qkv, beta, a, gate, dt_bias, A_log, norm_w, state, meta, H, G, d, dv, unit_eps, norm_eps,
+                         out_dtype):
+        """Gated delta rule with a decay per head and key channel.  qkv = [q (G d) | k (G d) | v (H dv)] as convolved; head h
+        reads q / k head h // (H / G).  Per head a state S carried transposed in ``state[slot]`` ([H, dv, d]):
+        S <- diag(g) S,  u = sigmoid(beta) (v - S^T k),  S <- S + k u^T,  o = S^T q  with q and k divided by sqrt(sum(x^2) +
+        unit_eps), q times d^(-1/2), g = exp(-exp(A_log[h]) softplus(a + dt_bias)).  Returns
+        o / sqrt(mean_head(o^2) + norm_eps) * norm_w * sigmoid(gate)  (norm_w [dv], shared by the heads)."""
+        T, rep = qkv.shape[0], H // G
+        f = qkv.float()
+        unit = lambda x: x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) + unit_eps)
+        q = (unit(f[:, :G * d].reshape(T, G, d)) * d ** -0.5).repeat_interleave(rep, 1)
+        k = unit(f[:, G * d:2 * G * d].reshape(T, G, d)).repeat_interleave(rep, 1)
+        v = f[:, 2 * G * d:].reshape(T, H, dv)
+        b = torch.sigmoid(beta.float())
+        g = torch.exp(-torch.exp(A_log.float())[None, :, None] * F.softplus(a.float() + dt_bias.float()).reshape(T, H, d))
+        o = torch.empty(T, H, dv, dtype=torch.float32, device=qkv.device)
+        cu, pos0, slot = meta["cu_host"], meta["pos0_host"], meta["slot"].tolist()
+        for s in range(len(slot)):
+            S = state[slot[s]].clone() if pos0[s] > 0 else torch.zeros(H, dv, d, device=qkv.device)
+            for t in range(int(cu[s]), int(cu[s + 1])):
+                S = S * g[t][:, None, :]
+                u = b[t][:, None] * (v[t] - torch.einsum("hvk,hk->hv", S, k[t]))
+                S = S + u[:, :, None] * k[t][:, None, :]
+                o[t] = torch.einsum("hvk,hk->hv", S, q[t])
+            state[slot[s]] = S
+        o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + norm_eps) * norm_w.float()
+        return (o.reshape(T, H * dv) * torch.sigmoid(gate.float())).to(out_dtype)
 
     def diff_combine(self, a, lam_w, diff, H, dv, eps, out_dtype):
         """a: [T, 2 H dv], the outputs of two score maps, all heads of the first map, then all of the second.
@@ -560,6 +634,32 @@ class TorchSeqOps:
             cand = torch.where(ok.repeat_interleave(per, 1), sc, torch.full_like(sc, -1.0))
         ids = torch.sort(cand, dim=-1, descending=True, stable=True).indices[:, :top]
         w = sc.gather(1, ids)
+        w = w / (w.sum(-1, keepdim=True) + 1e-20) * float(scale)
+        flat = ids.reshape(-1)
+        order = torch.sort(flat, stable=True).indices
+        dest = torch.empty_like(order)
+        dest[order] = torch.arange(order.numel(), device=order.device)
+        offs = torch.zeros(E + 1, dtype=torch.int32, device=logits.device)
+        offs[1:] = torch.cumsum(torch.bincount(flat, minlength=E), 0)
+        return SeqRoute(ids.int(), w, offs, (order // top).int(), dest.int().reshape(T, top), top)
+
+    def moe_route_softmax_grouped(self, logits, corr, top, groups, keep, scale):
+        """Scores s = softmax(logits), choice scores s + ``corr`` (None: s).  The experts form ``groups`` equal groups of
+        neighbours, a group is worth its largest choice score, only experts of the ``keep`` best groups compete (``groups`` 0
+        or 1: all do).  The ``top`` largest choice scores are chosen (ties: the lower expert), weighted by
+        s / (sum of the chosen s + 1e-20) * scale."""
+        T, E = logits.shape
+        s = torch.softmax(logits.float(), -1)
+        cand = s if corr is None else s + corr.float()
+        if groups and groups > 1:
+            per = E // groups
+            worth = cand.reshape(T, groups, per).max(-1).values
+            kept = torch.sort(worth, dim=-1, descending=True, stable=True).indices[:, :keep]
+            ok = torch.zeros(T, groups, dtype=torch.bool, device=logits.device)
+            ok.scatter_(1, kept, True)
+            cand = torch.where(ok.repeat_interleave(per, 1), cand, torch.full_like(cand, -math.inf))
+        ids = torch.sort(cand, dim=-1, descending=True, stable=True).indices[:, :top]
+        w = s.gather(1, ids)
         w = w / (w.sum(-1, keepdim=True) + 1e-20) * float(scale)
         flat = ids.reshape(-1)
         order = torch.sort(flat, stable=True).indices

@@ -457,6 +457,8 @@ class StepBatch:
     local_table: Optional[np.ndarray] = None
     # block length P -> [B, pages] int32 pages of the requests' key / value blocks (SequenceStateCache.block_table)
     block_tables: dict = field(default_factory=dict)
+    # [T] int32 token before each row's in its sequence (-1: none); only for stacks whose embedding reads it
+    prev_ids: Optional[np.ndarray] = None
     prompt_ids: List[int] = field(default_factory=lambda: [0])
     _dev: dict = field(default_factory=dict, repr=False)
 
@@ -478,6 +480,8 @@ class StepBatch:
             # one host-to-device copy for all the index arrays: each becomes a view of one int32 buffer
             # (segments padded to 16 entries, so every view starts 64-byte aligned)
             names = ["ids", "tok_seq", "tok_pos", "cu", "pos0", "slot", "page_table", "kv_slot", "want_idx"]
+            if self.prev_ids is not None:
+                names.append("prev_ids")
             if self.q_tiles is not None:
                 names += ["q_tiles", "tile_cu"]
             if self.local_table is not None:
@@ -501,7 +505,7 @@ class StepBatch:
 def pack_step(entries: Sequence[StepEntry], cache) -> StepBatch:
     """Pack one micro-batch of a step and claim its rows' places in ``cache`` (a
     runtime.seq_state.SequenceStateCache): pages for the new tokens, a state slot for a new request."""
-    ids, want, wc, cu, pos0, slot = [], [], [], [0], [], []
+    ids, want, wc, cu, pos0, slot, prev = [], [], [], [0], [], [], []
     ps = cache.page_size
     for e in entries:
         n = len(e.tokens)
@@ -511,6 +515,8 @@ def pack_step(entries: Sequence[StepEntry], cache) -> StepBatch:
         pos0.append(p0)
         slot.append(s)
         ids.append(np.asarray(e.tokens, dtype=np.int32))
+        if cache.prev_token:
+            prev += [np.asarray([cache.advance_token(e.rid, e.tokens[-1])], dtype=np.int32), ids[-1][:-1]]
         w = np.asarray(list(e.want), dtype=np.int64)
         if w.size and (w.min() < 0 or w.max() >= n):
             raise ValueError(f"request {e.rid!r}: a wanted place lies outside its {n} tokens")
@@ -537,7 +543,7 @@ def pack_step(entries: Sequence[StepEntry], cache) -> StepBatch:
         tile_cu = i32(np.concatenate([[0], np.cumsum([-(-(b - a) // Q_TILE_ROWS) for a, b in zip(cu[:-1], cu[1:])])]))
     return StepBatch(rids, i32(ids), i32(seq), i32(pos), i32(cu), i32(pos0), i32(slot), table,
                      i32(pages.astype(np.int64) * ps + pos_a % ps), i32(want), wc, len(ids), max_rows, q_tiles, tile_cu, local,
-                     {P: cache.block_table(rids, P) for P in cache.block_sizes})
+                     {P: cache.block_table(rids, P) for P in cache.block_sizes}, np.concatenate(prev) if prev else None)
 
 
 def split_step(entries: Sequence[StepEntry], token_budget: int) -> List[List[int]]:

@@ -271,6 +271,8 @@ class StepGraphs:
         m["page_table"] = self._widened(batch.page_table)
         for P, t in batch.block_tables.items():
             m[f"block_table_{P}"] = self._widened(t)
+        if batch.prev_ids is not None:
+            m["prev_ids"] = batch.prev_ids
         m["want_idx"] = np.arange(B, dtype=np.int32)
         return m
 

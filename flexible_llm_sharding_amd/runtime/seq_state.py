@@ -18,6 +18,7 @@ The scoring engine's :class:`~.prefix_cache.PrefixKVCache` keeps whole prefixes 
   ``taps - 1`` inputs of its short convolution.  A request holds one slot number, the same in every
   layer.  A request that starts at position 0 never reads its slot (the kernels start from zeros),
   so a slot or page that is handed out again needs no clearing;
+* a stack whose embedding looks at the token before has each request remember its last token;
 * attention that only looks inside the current chunk of the sequence (or a window) never reads
   older keys again: :meth:`trim` gives pages wholly behind every layer's horizon back to the pool
   (never the pages of the first tokens that a window keeps for good).
@@ -35,13 +36,14 @@ PAGE_SIZE = 16
 
 
 class _Request:
-    __slots__ = ("slot", "pages", "length", "first_page", "block_pages")
+    __slots__ = ("slot", "pages", "length", "first_page", "block_pages", "last_token")
 
     def __init__(self, slot: int):
         self.slot = slot
         self.pages: List[int] = []     # page numbers from logical page ``first_page`` on (-1: given back)
         self.length = 0                # tokens stored so far
         self.first_page = 0
+        self.last_token = -1           # (kept when the family's embedding reads the token before: ``prev_token``)
         self.block_pages: Dict[int, List[int]] = {}      # block length P -> pages of the request's blocks
 
 
@@ -57,6 +59,7 @@ class SequenceStateCache:
         #   horizons (kind, size, keep_first) of every layer that reads pages: "chunk": the keys of the
         #            current chunk of ``size`` positions; "window": the last ``size`` positions, and for
         #            good the first ``keep_first`` of the sequence
+        #   prev_token  whether the embedding of a token reads the one before it
         from ..models import hybrid_family
         spec = hybrid_family(cfg).state_spec(cfg)
         self.attn: Dict[str, dict] = dict(spec["paged"])
@@ -65,6 +68,7 @@ class SequenceStateCache:
         self.block_sizes = sorted({P for P, _ in self.blocks.values()})
         self.rec: Dict[str, dict] = dict(spec["slots"])
         self.horizons = list(spec["horizons"])
+        self.prev_token = bool(spec.get("prev_token", False))
         self.keep_pages = max([-(-int(k) // self.page_size) for _, _, k in self.horizons] + [0])
         self._kv: Dict[str, Dict[str, torch.Tensor]] = {}
         self._rec: Dict[str, Dict[str, torch.Tensor]] = {}
@@ -186,6 +190,12 @@ class SequenceStateCache:
                 mine.append(p)
         r.length = pos0 + n_tokens
         return pos0, r.slot
+
+    def advance_token(self, rid, last: int) -> int:
+        """The token before the request's rows of this step (-1: none); ``last``, their last one, takes its place."""
+        r = self.requests[rid]
+        prev, r.last_token = r.last_token, int(last)
+        return prev
 
     def horizon(self, next_pos: int) -> int:
         """First position past the kept first tokens that any layer can still read once the token at
