@@ -15,10 +15,11 @@ int fls_seq_version(void);
 // groups > 1 with offs == null: strided batch g: A + (g % a_mod) * a_gs, W + g * w_gs, C / bias + g * c_gs.
 // offs != null: row groups: group g owns rows [offs[g], offs[g+1]) of A and C and weight W + g * w_gs;
 // M is then the total row count (the bound of every group's rows).
-// Epilogue: + bias, then an activation (act_kind 0: none; 1: xIELU, act = {p, q} on the device; 2: max(z, 0)^2), stored as type tc (fp32, or bf16 when the
+// Epilogue: + bias, then an activation (act_kind 0: none; 1: xIELU, act = {p, q} on the device; 2: max(z, 0)^2;
+// 3: exp(-exp(act[n / act_n]) softplus(z)), a decay per column n; groups == 1), stored as type tc (fp32, or bf16 when the
 // consumer is the next product).
 int fls_seq_gemm(const void* A, int ta, const void* W, int tw, void* C, int tc, const float* bias, const float* act,
-                 int act_kind, int M, int N, int K, int lda, int ldw, int ldc, int groups, const int* offs, long long a_gs,
+                 int act_kind, int act_n, int M, int N, int K, int lda, int ldw, int ldc, int groups, const int* offs, long long a_gs,
                  int a_mod, long long w_gs, long long c_gs, fls_stream_t s);
 // y[r] = w * x[row] / sqrt(mean_g(x[row]^2) + eps) per group of D / groups columns, row = idx ? idx[r] : r.
 // add != 0: y (fp32) += instead (the residual update), ty ignored.  woff is added to the weight (1 for
@@ -43,8 +44,10 @@ int fls_seq_add_scaled(float* x, int ldx, const float* y, int ldy, int rows, int
 int fls_seq_gather_rows(const void* x, int tx, int ldx, const int* idx, void* y, int ldy, int rows, int D, fls_stream_t s);
 // xIELU: z > 0: softplus(p) z^2 + z/2; else (1/2 + softplus(q)) (exp(z) - 1 - z) + z/2; act = {p, q}
 int fls_seq_xielu(const float* z, int ldz, const float* act, void* y, int ty, int ldy, int rows, int cols, fls_stream_t s);
-// y[r, c] = act(gu[r, c]) * gu[r, cols + c]; act: 0 = silu, 1 = gelu (tanh form)
-int fls_seq_gate_mul(const float* gu, int ldg, void* y, int ty, int ldy, int rows, int cols, int act, fls_stream_t s);
+// y[r, c] = act(gu[r, c]) * gu[r, cols + c]; act: 0 = silu, 1 = gelu (tanh form), 2 = clamped: with g = min(gu[r, c], limit)
+// and u = clamp(gu[r, cols + c], -limit, limit): g sigmoid(alpha g) (u + 1)
+int fls_seq_gate_mul(const float* gu, int ldg, void* y, int ty, int ldy, int rows, int cols, int act, float limit, float alpha,
+                     fls_stream_t s);
 // y = f(z) elementwise; kind: 0 = tanh, 1 = gelu (exact: 0.5 z (1 + erf(z / sqrt 2))), 2 = z (a cast)
 int fls_seq_unary(const float* z, int ldz, void* y, int ty, int ldy, int rows, int cols, int kind, fls_stream_t s);
 // per row t and head h: the n entries x[t, x_col + h x_hs ...] (x of type tx), RMS-normed over n times w[n] (w != null), the first
@@ -71,7 +74,7 @@ int fls_seq_kv_store(const float* k, int ldk, const float* kn, float eps, const 
 // pools and out of type tc.  out = result * out_scale.  nsplit > 1: every row's keys are cut into nsplit
 // ranges that run as blocks of their own (few rows, many keys: decoding) and are merged by a second
 // kernel; part: T H nsplit (dv + 4) floats of scratch (16-byte aligned).  has_sink != 0 (softmax only): one more
-// entry of score `sink` and no value joins the softmax's sum.  head_gate (nullable) [T, H] fp32, row stride ldhg:
+// entry of score `sink` (sink_h given: of score sink_h[h]) and no value joins the softmax's sum.  head_gate (nullable) [T, H] fp32, row stride ldhg:
 // the output of (row, head) times sigmoid(head_gate[t, h]).
 // out of type to (fp32 over bf16 pools allowed).  Gv (0: G), a divisor of G: the value pool holds Gv heads and key head g
 // reads value head g % Gv (several score maps over the same values).
@@ -83,8 +86,8 @@ int fls_seq_attn_paged(const void* q, int ldq, int tq, const void* kc, int ldk, 
                        int pt_stride, int T, int H, int G, int d, int dv, float scale, float softcap,
                        const float* r1, const float* r2, int chunk, int window, int keep_first,
                        const float* gate_bias, float out_scale, int page_size, int nsplit, float* part,
-                       int has_sink, float sink, const float* head_gate, int ldhg, int Gv, int pool_P, const void* kp,
-                       int ldkp, const void* vp, int ldvp, const int* block_table, int bt_stride, fls_stream_t s);
+                       int has_sink, float sink, const float* sink_h, const float* head_gate, int ldhg, int Gv,
+                       int pool_P, const void* kp, int ldkp, const void* vp, int ldvp, const int* block_table, int bt_stride, fls_stream_t s);
 // the same attention on the matrix cores for bf16 pools and rows in tiles: tiles[n_tiles][2] = (first packed
 // row, rows <= 128) of one request each, covering every row of the step; q of type tq.  -2: shape not
 // served (use the above)
@@ -92,16 +95,16 @@ int fls_seq_attn_prefill(const void* q, int ldq, int tq, const void* kc, int ldk
                          int to, int ldo, const int* tiles, int n_tiles, const int* tok_seq, const int* tok_pos,
                          const int* page_table, int pt_stride, int H, int G, int d, int dv, float scale,
                          float softcap, const float* r1, const float* r2, int chunk, int window, int keep_first,
-                         const float* gate_bias, float out_scale, int page_size, int has_sink, float sink,
+                         const float* gate_bias, float out_scale, int page_size, int has_sink, float sink, const float* sink_h,
                          const float* head_gate, int ldhg, int Gv, int pool_P, const void* kp, int ldkp, const void* vp,
                          int ldvp, const int* block_table, int bt_stride, fls_stream_t s);
 // softmax attention of few rows whose H / G <= 32 query heads per key / value head become the columns of one
 // matrix-core tile (decode steps over cached latent rows): fp32 q, bf16 pools and out, window and kept first
-// keys as above; nsplit ranges of key tiles per row, part: T H nsplit (dv + 4) floats.  -2: shape not served
+// keys, sink_h[H] and head_gate as above (nullable); nsplit ranges of key tiles per row, part: T H nsplit (dv + 4) floats.  -2: shape not served
 int fls_seq_attn_heads(const void* q, int ldq, const void* kc, int ldk, const void* vc, int ldv, void* out, int ldo,
                        const int* tok_seq, const int* tok_pos, const int* page_table, int pt_stride, int T, int H,
                        int G, int d, int dv, float scale, int window, int keep_first, float out_scale, int page_size,
-                       int nsplit, float* part, fls_stream_t s);
+                       int nsplit, float* part, const float* sink_h, const float* head_gate, int ldhg, fls_stream_t s);
 // causal per-channel convolution over each request's rows, history from / to state[slot][taps-1][C];
 // b nullable; residual != 0: + the input row; out of type to; one_row_each != 0: the caller knows that every
 // request brings exactly one row (the state is then rewritten by the same kernel)
@@ -167,6 +170,13 @@ int fls_seq_moe_route(const float* logits, int ldl, const float* corr, int T, in
 // lower expert), w = score / (sum of the chosen + 1e-20) * scale; hist as above.  groups <= 64
 int fls_seq_moe_route_grouped(const float* logits, int ldl, int T, int E, int top, int groups, int keep, float scale,
                               int* ids, float* w, int* hist, fls_stream_t s);
+// scores s = softmax(logits) over all E outputs, choice scores s + corr (corr nullable); `groups` equal groups of neighbours,
+// each worth its largest choice score, only the `keep` best groups compete (groups <= 1: all); the top largest choice scores are
+// chosen (ties: the lower index), w = s / (sum of the chosen s + 1e-20) * scale.  T <= FLS_SEQ_ROUTE_FUSED: the same launch also
+// sorts the entries by expert (offs[E + 1], dest[T, top], rows[T top]); otherwise hist as above and those three are left alone
+#define FLS_SEQ_ROUTE_FUSED 64
+int fls_seq_moe_route_softmax_grouped(const float* logits, int ldl, const float* corr, int T, int E, int top, int groups, int keep,
+                                      float scale, int* ids, float* w, int* hist, int* offs, int* dest, int* rows, fls_stream_t s);
 // offs[E+1] = exclusive scan of hist; cursor[E] = offs[:E]
 int fls_seq_moe_scan(const int* hist, int E, int* offs, int* cursor, fls_stream_t s);
 // dest[t, k] = a row in its expert's range; rows[dest] = t
@@ -178,9 +188,11 @@ int fls_seq_moe_sum(const float* y, int ldy, const int* dest, const float* w, fl
 int fls_seq_moe_combine(float* x, int ldx, const float* y, int ldy, const int* dest, const float* w, int T, int top,
                         const float* shared, int lds, const float* gate, int ldg, int D, float mult, fls_stream_t s);
 // ---- several residual streams per row (streams.hip).  xs: fp32 [rows, S D], a row's S streams side by side
-// out[t, c * D ...] = table[ids[t]] * scale + pos_table[tok_pos[t]] (pos_table nullable; positions clamped to P - 1), c < copies
-int fls_seq_embed_pos(const int* ids, const void* table, int tt, const void* pos_table, const int* tok_pos, float* out, int T,
-                      int D, int V, int P, float scale, int copies, fls_stream_t s);
+// out[t, c * D ...] = table[ids[t]] * scale + pos_table[tok_pos[t]] (pos_table nullable; positions clamped to P - 1)
+// + pair_table[(prev[t] mul_prev + ids[t] mul_cur) mod buckets] (pair_table nullable; prev[t] < 0: its row `buckets`), c < copies
+int fls_seq_embed_pos(const int* ids, const void* table, int tt, const void* pos_table, const int* tok_pos, const void* pair_table,
+                      const int* prev, int buckets, long long mul_prev, long long mul_cur, float* out, int T, int D, int V, int P,
+                      float scale, int copies, fls_stream_t s);
 // u = sum_s coef[s] xs[row, s] (coef nullable: the plain sum), y[r] = u / sqrt(mean(u^2) + eps) * w; row = idx ? idx[r] : r
 int fls_seq_streams_norm(const float* xs, int ldx, const int* idx, const float* coef, const float* w, void* y, int ty, int ldy,
                          int rows, int D, int S, float eps, fls_stream_t s);
@@ -204,6 +216,30 @@ int fls_seq_diff_combine(const float* a, int lda, const float* lam_w, int d, flo
 int fls_seq_hgrn2_scan(const float* q, int ldq, const float* f, int ldf, const float* v, int ldv, const float* fb,
                        const float* lower, float* state, float* raw, int ldo, const int* cu, const int* pos0,
                        const int* slot, int B, int H, int d, int dv, fls_stream_t s);
+// ---- layers whose sublayers run side by side (parallel.hip)
+// two norms of one row: h1 = x rs w1, h2 = x rs w2 (w2 / h2 nullable), rs = 1 / sqrt(mean(x^2) + eps); add (nullable): x += add first
+int fls_seq_rmsnorm_pair(float* x, int ldx, const float* add, int ldadd, const float* w1, void* h1, int ld1, const float* w2, void* h2,
+                         int ld2, int th, int rows, int D, float eps, fls_stream_t s);
+// x += a wa + f wb (fp32 rows, one number per column in wa / wb).  f = b; or, with dest != null, the experts' sum
+// sum_k w[t, k] (ids[t, k] < E ? y[dest[t, k]] : h[t]) (h of type th); or, with neither, nothing
+int fls_seq_parallel_update(float* x, int ldx, const float* a, int lda, const float* wa, const float* b, int ldb, const float* wb,
+                            const float* y, int ldy, const int* dest, const float* w, const int* ids, int top, int E, const void* h,
+                            int th, int ldh, int rows, int D, fls_stream_t s);
+// rows z = [query latent (qr) | latent (r) | rotated key part (dr) | ...] of a latent attention: cq = rms(query latent) qw (qr = 0:
+// none), row kv_slot[t] of the pool (pw wide) = [rms(latent) kw | key part rotated in pairs (i, i + rot / 2), angle
+// tok_pos freqs[i]]; cq and the pool of type tp
+int fls_seq_latent_rows(const float* z, int ldz, int qr, int r, int dr, const float* qw, const float* kw, float eps,
+                        const float* freqs, int rot, const int* tok_pos, const int* kv_slot, void* cq, int ldcq, void* pool, int pw,
+                        int tp, int T, fls_stream_t s);
+// ---- gated delta rule with a decay per key channel (gated_delta.hip).  Per head a state S[d][dv], kept transposed in
+// state[slot][H][dv][d]: S <- diag(g) S; u = sigmoid(beta) (v - S^T k); S <- S + k u^T; o = S^T q.  qkv = fp32 rows
+// [q (G d) | k (G d) | v (H dv)], head h reads q / k head h / (H / G); q and k are divided by sqrt(sum(x^2) + unit_eps), q times
+// q_scale; decay: fp32 [T, H d] in (0, 1]; out = o / sqrt(mean_head(o^2) + norm_eps) norm_w sigmoid(gate).  d <= 256, dv <= 512.
+// raw: T H dv floats of scratch (16-byte aligned)
+int fls_seq_gated_delta_scan(const float* qkv, int ldq, const float* beta, int ldb, const float* decay, int ldd, const float* gate,
+                             int ldg, const float* norm_w, float* state, float* raw, void* out, int to, int ldo, const int* cu,
+                             const int* pos0, const int* slot, int T, int B, int one_row_each, int H, int G, int d, int dv,
+                             float q_scale, float unit_eps, float norm_eps, fls_stream_t s);
 #ifdef __cplusplus
 }
 #endif

@@ -4,7 +4,7 @@
 // keep_first keys of the sequence however far back they lie.  Keys and values are the first G d and
 // G dv columns of pool rows ldk and ldv wide, so both may be one pool (values = a prefix of the keys:
 // attention over latent rows).  The query may be fp32 while the pools hold bf16.  has_sink: the softmax
-// has one more entry of score `sink` and no value (p_j = exp(s_j) / (exp(sink) + sum exp(s))); head_gate
+// has one more entry of score `sink` (sink_h given: sink_h[head]) and no value (p_j = exp(s_j) / (exp(sink) + sum exp(s))); head_gate
 // [T, H] fp32: the output of (row, head) times sigmoid(head_gate[t, h]).  Pooled blocks (pool_P > 0, beside a window):
 // the softmax also runs over one mean key and value for each block of pool_P positions that ends before the window,
 // read from block pools with pages of their own.
@@ -61,7 +61,8 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
                                                          int chunk, int window, int keep_first,
                                                          const float* __restrict__ gate_bias, float out_scale,
                                                          int page_size, int vec, float* __restrict__ part, int has_sink,
-                                                         float sink, const float* __restrict__ head_gate, int ldhg, int Gv,
+                                                         float sink, const float* __restrict__ sink_h,
+                                                         const float* __restrict__ head_gate, int ldhg, int Gv,
                                                          AttnBlocks ab) {
   __shared__ float qs[MAX_D];
   __shared__ float pw[4][64];
@@ -88,6 +89,7 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
   const float a1 = r1 != nullptr ? r1[h] : 0.f, a2 = r2 != nullptr ? r2[h] : 0.f;
   const bool gated = gate_bias != nullptr;
   const float gb = gated ? gate_bias[h] : 0.f;
+  const float snk = has_sink && sink_h != nullptr ? sink_h[h] : sink;
   float m = -1e30f, l = 0.f;
   float acc[MAX_DV_PER_LANE];
 #pragma unroll
@@ -162,10 +164,10 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
       for (int w = 0; w < 4; ++w) f[w] = 1.f;
     } else {
       mx = fmaxf(fmaxf(mm[0], mm[1]), fmaxf(mm[2], mm[3]));
-      if (has_sink && nsplit == 1) mx = fmaxf(mx, sink);          // (with ranges the merge adds the silent entry, once)
+      if (has_sink && nsplit == 1) mx = fmaxf(mx, snk);           // (with ranges the merge adds the silent entry, once)
 #pragma unroll
       for (int w = 0; w < 4; ++w) { f[w] = expf(mm[w] - mx); lt += ll[w] * f[w]; }
-      if (has_sink && nsplit == 1) lt += expf(sink - mx);
+      if (has_sink && nsplit == 1) lt += expf(snk - mx);
       inv = out_scale / lt;
     }
     if (head_gate != nullptr) inv *= sigmoid_f(head_gate[(size_t)t * ldhg + h]);
@@ -196,7 +198,8 @@ __global__ __launch_bounds__(256) void attn_paged_kernel(const TQ* __restrict__ 
 #define MERGE_MAX_SPLIT 64
 template <typename T>
 __global__ void attn_merge_kernel(const float* __restrict__ part, T* __restrict__ out, int ldo, int H, int dv, int nsplit, int gated,
-                                  float out_scale, int has_sink, float sink, const float* __restrict__ head_gate, int ldhg) {
+                                  float out_scale, int has_sink, float sink, const float* __restrict__ sink_h,
+                                  const float* __restrict__ head_gate, int ldhg) {
   __shared__ float wz[MERGE_MAX_SPLIT];
   const int t = blockIdx.y, h = blockIdx.x;
   const int rs = dv + 4;                           // record: values[dv] | maximum | sum | pad
@@ -206,10 +209,11 @@ __global__ void attn_merge_kernel(const float* __restrict__ part, T* __restrict_
     const float mz = (z < nsplit && !gated) ? pp[z * rs + dv] : -1e30f;
     const float lz = (z < nsplit && !gated) ? pp[z * rs + dv + 1] : 0.f;
     float mx = wave_max(mz);
-    if (has_sink) mx = fmaxf(mx, sink);
+    const float snk = has_sink && sink_h != nullptr ? sink_h[h] : sink;
+    if (has_sink) mx = fmaxf(mx, snk);
     const float f = expf(mz - mx);
     float lt = wave_sum(lz * f);
-    if (has_sink) lt += expf(sink - mx);
+    if (has_sink) lt += expf(snk - mx);
     const float os = head_gate != nullptr ? out_scale * sigmoid_f(head_gate[(size_t)t * ldhg + h]) : out_scale;
     wz[z] = gated ? os : f * os / lt;
   }
@@ -223,11 +227,11 @@ __global__ void attn_merge_kernel(const float* __restrict__ part, T* __restrict_
 
 // (also used by the matrix-core kernels that cut a row's keys over blocks)
 int seq_attn_merge(const float* part, void* out, int tc, int ldo, int T, int H, int dv, int nsplit, int gated, float out_scale,
-                   int has_sink, float sink, const float* head_gate, int ldhg, fls_stream_t s) {
+                   int has_sink, float sink, const float* sink_h, const float* head_gate, int ldhg, fls_stream_t s) {
   const int threads = dv > 128 ? 256 : (dv > 64 ? 128 : 64);
   hipStream_t st = (hipStream_t)s;
-  if (tc == 1) hipLaunchKernelGGL((attn_merge_kernel<bf16_t>), dim3(H, T), dim3(threads), 0, st, part, (bf16_t*)out, ldo, H, dv, nsplit, gated, out_scale, has_sink, sink, head_gate, ldhg);
-  else hipLaunchKernelGGL((attn_merge_kernel<float>), dim3(H, T), dim3(threads), 0, st, part, (float*)out, ldo, H, dv, nsplit, gated, out_scale, has_sink, sink, head_gate, ldhg);
+  if (tc == 1) hipLaunchKernelGGL((attn_merge_kernel<bf16_t>), dim3(H, T), dim3(threads), 0, st, part, (bf16_t*)out, ldo, H, dv, nsplit, gated, out_scale, has_sink, sink, sink_h, head_gate, ldhg);
+  else hipLaunchKernelGGL((attn_merge_kernel<float>), dim3(H, T), dim3(threads), 0, st, part, (float*)out, ldo, H, dv, nsplit, gated, out_scale, has_sink, sink, sink_h, head_gate, ldhg);
   SEQ_LAUNCH_CHECK();
   return 0;
 }
@@ -238,7 +242,7 @@ extern "C" int fls_seq_attn_paged(const void* q, int ldq, int tq, const void* kc
                                   int pt_stride, int T, int H, int G, int d, int dv, float scale, float softcap,
                                   const float* r1, const float* r2, int chunk, int window, int keep_first,
                                   const float* gate_bias, float out_scale, int page_size, int nsplit, float* part,
-                                  int has_sink, float sink, const float* head_gate, int ldhg, int Gv, int pool_P, const void* kp,
+                                  int has_sink, float sink, const float* sink_h, const float* head_gate, int ldhg, int Gv, int pool_P, const void* kp,
                                   int ldkp, const void* vp, int ldvp, const int* block_table, int bt_stride, fls_stream_t s) {
   if (T <= 0) return 0;
   if (Gv <= 0) Gv = G;
@@ -254,7 +258,7 @@ extern "C" int fls_seq_attn_paged(const void* q, int ldq, int tq, const void* kc
   dim3 grid(H, T, nsplit);
   hipStream_t st = (hipStream_t)s;
 #define ATTN_PAGED_ARGS ldq, (const TC*)kc, ldk, (const TC*)vc, ldv, (TOUT*)out, ldo, tok_seq, tok_pos, page_table, pt_stride, H, G, \
-                        d, dv, scale, softcap, r1, r2, chunk, window, keep_first, gate_bias, out_scale, page_size, vec, part, has_sink, sink, \
+                        d, dv, scale, softcap, r1, r2, chunk, window, keep_first, gate_bias, out_scale, page_size, vec, part, has_sink, sink, sink_h, \
                         nsplit > 1 ? nullptr : head_gate, ldhg, Gv, ab
 #define ATTN_PAGED_GO(TQ)                                                                                                   \
   do {                                                                                                                      \
@@ -282,6 +286,6 @@ extern "C" int fls_seq_attn_paged(const void* q, int ldq, int tq, const void* kc
 #undef ATTN_PAGED_GO
 #undef ATTN_PAGED_ARGS
   SEQ_LAUNCH_CHECK();
-  if (nsplit > 1) return seq_attn_merge(part, out, to, ldo, T, H, dv, nsplit, gate_bias != nullptr, out_scale, has_sink, sink, head_gate, ldhg, s);
+  if (nsplit > 1) return seq_attn_merge(part, out, to, ldo, T, H, dv, nsplit, gate_bias != nullptr, out_scale, has_sink, sink, sink_h, head_gate, ldhg, s);
   return 0;
 }

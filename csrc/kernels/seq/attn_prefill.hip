@@ -41,7 +41,8 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_kernel(const TQ* __restri
                                                            const float* __restrict__ r1, const float* __restrict__ r2,
                                                            int chunk, int window, int keep_first,
                                                            const float* __restrict__ gate_bias, float out_scale, int page_size,
-                                                           int has_sink, float sink, const float* __restrict__ head_gate,
+                                                           int has_sink, float sink, const float* __restrict__ sink_h,
+                                                           const float* __restrict__ head_gate,
                                                            int ldhg, int Gv, AttnBlocks ab) {
   constexpr int KLD = D + 8;
   __shared__ __attribute__((aligned(16))) bf16_t Ks[KT * KLD];
@@ -89,8 +90,8 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_kernel(const TQ* __restri
   for (int c = 0; c < DV / 32; ++c)
 #pragma unroll
     for (int r = 0; r < 16; ++r) O[c][r] = 0.f;
-  // (the softmax's silent entry of score `sink`, if any, is where every query's running maximum and sum start)
-  float m = has_sink ? sink : -1e30f, l = has_sink ? 1.f : 0.f;
+  // (the softmax's silent entry of score `sink` / sink_h[h], if any, is where every query's running maximum and sum start)
+  float m = has_sink ? (sink_h != nullptr ? sink_h[h] : sink) : -1e30f, l = has_sink ? 1.f : 0.f;
   const float a1 = r1 != nullptr ? r1[h] : 0.f, a2 = r2 != nullptr ? r2[h] : 0.f;
   const bool gated = gate_bias != nullptr;
   const float gb = gated ? gate_bias[h] : 0.f;
@@ -261,7 +262,7 @@ extern "C" int fls_seq_attn_prefill(const void* q, int ldq, int tq, const void* 
                                     int to, int ldo, const int* tiles, int n_tiles, const int* tok_seq, const int* tok_pos,
                                     const int* page_table, int pt_stride, int H, int G, int d, int dv, float scale,
                                     float softcap, const float* r1, const float* r2, int chunk, int window, int keep_first,
-                                    const float* gate_bias, float out_scale, int page_size, int has_sink, float sink,
+                                    const float* gate_bias, float out_scale, int page_size, int has_sink, float sink, const float* sink_h,
                                     const float* head_gate, int ldhg, int Gv, int pool_P, const void* kp, int ldkp, const void* vp,
                                     int ldvp, const int* block_table, int bt_stride, fls_stream_t s) {
   if (n_tiles <= 0) return 0;
@@ -281,7 +282,7 @@ extern "C" int fls_seq_attn_prefill(const void* q, int ldq, int tq, const void* 
   hipLaunchKernelGGL((attn_prefill_kernel<DD, DDV, TQ_, TO_, PP>), grid, dim3(256), 0, st, (const TQ_*)q, ldq,            \
                      (const bf16_t*)kc, ldk, (const bf16_t*)vc, ldv, (TO_*)out, ldo, tiles, tok_seq, tok_pos,             \
                      page_table, pt_stride, H, G, scale, softcap, r1, r2, chunk, window, keep_first, gate_bias,           \
-                     out_scale, page_size, has_sink, sink, head_gate, ldhg, Gv, ab)
+                     out_scale, page_size, has_sink, sink, sink_h, head_gate, ldhg, Gv, ab)
 #define ATTN_PF(DD, DDV)                                                                                                  \
   do {                                                                                                                    \
     if (tq == 1 && to == 1) ATTN_PF_(DD, DDV, bf16_t, bf16_t, false);                                                     \
@@ -329,7 +330,8 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(const float* __restrict
                                                          const int* __restrict__ tok_seq, const int* __restrict__ tok_pos,
                                                          const int* __restrict__ page_table, int pt_stride, int H, int G,
                                                          float scale, int window, int keep_first, float out_scale,
-                                                         int page_size, float* __restrict__ part) {
+                                                         int page_size, float* __restrict__ part, const float* __restrict__ sink_h,
+                                                         const float* __restrict__ head_gate, int ldhg) {
   constexpr int KLD = D + 8;
   constexpr int CPW = DV / 128;               // 32-column blocks of the values per wave
   __shared__ __attribute__((aligned(16))) bf16_t Ks[KT * KLD];
@@ -370,7 +372,9 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(const float* __restrict
   for (int c = 0; c < CPW; ++c)
 #pragma unroll
     for (int r = 0; r < 16; ++r) O[c][r] = 0.f;
-  float m = -1e30f, l = 0.f;
+  // (a silent softmax entry of score sink_h[head] is where the running maximum and sum start; with ranges the merge adds it)
+  const bool snk = sink_h != nullptr && nsplit == 1;
+  float m = snk ? sink_h[head] : -1e30f, l = snk ? 1.f : 0.f;
   constexpr int NK = KT * (D / 8) / 256, NV = KT * (DV / 8) / 256;
   static_assert(NK >= 1 && NV >= 1 && KT * (D / 8) % 256 == 0 && KT * (DV / 8) % 256 == 0 && CPW >= 1, "tile pieces per thread");
   uint4 kreg[NK], vreg[NV];
@@ -481,7 +485,8 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(const float* __restrict
   }
   if (!qok) return;
   if (nsplit == 1) {
-    const float inv = out_scale / l;
+    float inv = out_scale / l;
+    if (head_gate != nullptr) inv *= sigmoid_f(head_gate[(size_t)t * ldhg + head]);
     bf16_t* op = out + (size_t)t * ldo + (size_t)head * DV;
 #pragma unroll
     for (int c = 0; c < CPW; ++c)
@@ -508,7 +513,7 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(const float* __restrict
 extern "C" int fls_seq_attn_heads(const void* q, int ldq, const void* kc, int ldk, const void* vc, int ldv, void* out, int ldo,
                                   const int* tok_seq, const int* tok_pos, const int* page_table, int pt_stride, int T, int H,
                                   int G, int d, int dv, float scale, int window, int keep_first, float out_scale, int page_size,
-                                  int nsplit, float* part, fls_stream_t s) {
+                                  int nsplit, float* part, const float* sink_h, const float* head_gate, int ldhg, fls_stream_t s) {
   if (T <= 0) return 0;
   if (G < 1 || H % G || H / G > 32 || page_size < 1 || nsplit < 1 || nsplit > 64 || (nsplit > 1 && part == nullptr) || ldq % 4 || ldo % 4 ||
       ldk % 8 || ldv % 8 || G * d > ldk || G * dv > ldv || (uintptr_t)q % 16 || (uintptr_t)kc % 16 || (uintptr_t)vc % 16 ||
@@ -519,13 +524,16 @@ extern "C" int fls_seq_attn_heads(const void* q, int ldq, const void* kc, int ld
 #define ATTN_HEADS(DD, DDV)                                                                                                \
   hipLaunchKernelGGL((attn_heads_kernel<DD, DDV>), grid, dim3(256), 0, st, (const float*)q, ldq, (const bf16_t*)kc, ldk,    \
                      (const bf16_t*)vc, ldv, (bf16_t*)out, ldo, tok_seq, tok_pos, page_table, pt_stride, H, G, scale, window, \
-                     keep_first, out_scale, page_size, part)
+                     keep_first, out_scale, page_size, part, sink_h, head_gate, ldhg)
   if (d == 576 && dv == 512) ATTN_HEADS(576, 512);
+  else if (d == 512 && dv == 512) ATTN_HEADS(512, 512);
+  else if (d == 256 && dv == 256) ATTN_HEADS(256, 256);
+  else if (d == 128 && dv == 128) ATTN_HEADS(128, 128);
   else if (d == 320 && dv == 256) ATTN_HEADS(320, 256);
   else if (d == 192 && dv == 128) ATTN_HEADS(192, 128);
   else return -2;
 #undef ATTN_HEADS
   SEQ_LAUNCH_CHECK();
-  if (nsplit > 1) return seq_attn_merge(part, out, 1, ldo, T, H, dv, nsplit, 0, out_scale, 0, 0.f, nullptr, 0, s);
+  if (nsplit > 1) return seq_attn_merge(part, out, 1, ldo, T, H, dv, nsplit, 0, out_scale, sink_h != nullptr, 0.f, sink_h, head_gate, ldhg, s);
   return 0;
 }

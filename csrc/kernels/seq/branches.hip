@@ -3,36 +3,10 @@
 //   new = (keep ? x : 0) + coef (rms(a) wa + rms(b) wb) + f;   x <- new;   h = rms(new) hw
 // (a, b, f and h each optional; hw is a vector, or one number for all columns).  All sums fp32.
 #include "seq_common.h"
+#include "row_vec.h"
 #include "fls_seq.h"
 
 #define RB_PIECES 8                // 256 VE columns a piece; that many pieces of a and b stay in registers
-
-template <int VE> struct RbVec { float v[VE]; };
-template <int VE>
-__device__ __forceinline__ RbVec<VE> rb_load(const float* p) {
-  RbVec<VE> r;
-  if constexpr (VE == 4) {
-    const float4 q = *reinterpret_cast<const float4*>(p);
-    r.v[0] = q.x; r.v[1] = q.y; r.v[2] = q.z; r.v[3] = q.w;
-  } else {
-    r.v[0] = p[0];
-  }
-  return r;
-}
-template <int VE>
-__device__ __forceinline__ void rb_store(float* p, const RbVec<VE>& r) {
-  if constexpr (VE == 4) *reinterpret_cast<float4*>(p) = make_float4(r.v[0], r.v[1], r.v[2], r.v[3]);
-  else p[0] = r.v[0];
-}
-template <int VE>
-__device__ __forceinline__ void rb_store(bf16_t* p, const RbVec<VE>& r) {
-  if constexpr (VE == 4) {
-    const bf16_t e[4] = {f_to_bf16(r.v[0]), f_to_bf16(r.v[1]), f_to_bf16(r.v[2]), f_to_bf16(r.v[3])};
-    *reinterpret_cast<uint2*>(p) = *reinterpret_cast<const uint2*>(e);
-  } else {
-    p[0] = f_to_bf16(r.v[0]);
-  }
-}
 
 // one block per row
 template <typename TO, int VE>
@@ -49,7 +23,7 @@ __global__ __launch_bounds__(256) void residual_branches_kernel(float* __restric
   const float* br = a != nullptr ? b + (size_t)r * ldb : nullptr;
   const float* fr = f != nullptr ? f + (size_t)r * ldf_ : nullptr;
   const int np = (D + 256 * VE - 1) / (256 * VE);
-  RbVec<VE> av[RB_PIECES], bv[RB_PIECES];
+  RowVec<VE> av[RB_PIECES], bv[RB_PIECES];
   float rsa = 0.f, rsb = 0.f;
   if (ar != nullptr) {
     float sa = 0.f, sb = 0.f;
@@ -57,8 +31,8 @@ __global__ __launch_bounds__(256) void residual_branches_kernel(float* __restric
     for (int k = 0; k < RB_PIECES; ++k) {
       const int c = (threadIdx.x + 256 * k) * VE;
       if (c < D) {
-        av[k] = rb_load<VE>(ar + c);
-        bv[k] = rb_load<VE>(br + c);
+        av[k] = row_load<VE>(ar + c);
+        bv[k] = row_load<VE>(br + c);
 #pragma unroll
         for (int i = 0; i < VE; ++i) { sa += av[k].v[i] * av[k].v[i]; sb += bv[k].v[i] * bv[k].v[i]; }
       }
@@ -66,7 +40,7 @@ __global__ __launch_bounds__(256) void residual_branches_kernel(float* __restric
     for (int k = RB_PIECES; k < np; ++k) {
       const int c = (threadIdx.x + 256 * k) * VE;
       if (c < D) {
-        const RbVec<VE> ta = rb_load<VE>(ar + c), tb = rb_load<VE>(br + c);
+        const RowVec<VE> ta = row_load<VE>(ar + c), tb = row_load<VE>(br + c);
 #pragma unroll
         for (int i = 0; i < VE; ++i) { sa += ta.v[i] * ta.v[i]; sb += tb.v[i] * tb.v[i]; }
       }
@@ -81,24 +55,24 @@ __global__ __launch_bounds__(256) void residual_branches_kernel(float* __restric
   }
   float ss = 0.f;
   // one piece of the row; returns the new entries
-  auto piece = [&](int c, const RbVec<VE>& pa, const RbVec<VE>& pb) -> RbVec<VE> {
-    RbVec<VE> n;
-    if (keep) n = rb_load<VE>(xr + c);
+  auto piece = [&](int c, const RowVec<VE>& pa, const RowVec<VE>& pb) -> RowVec<VE> {
+    RowVec<VE> n;
+    if (keep) n = row_load<VE>(xr + c);
     else {
 #pragma unroll
       for (int i = 0; i < VE; ++i) n.v[i] = 0.f;
     }
     if (ar != nullptr) {
-      const RbVec<VE> qa = rb_load<VE>(wa + c), qb = rb_load<VE>(wb + c);
+      const RowVec<VE> qa = row_load<VE>(wa + c), qb = row_load<VE>(wb + c);
 #pragma unroll
       for (int i = 0; i < VE; ++i) n.v[i] += pa.v[i] * rsa * qa.v[i] + pb.v[i] * rsb * qb.v[i];
     }
     if (fr != nullptr) {
-      const RbVec<VE> q = rb_load<VE>(fr + c);
+      const RowVec<VE> q = row_load<VE>(fr + c);
 #pragma unroll
       for (int i = 0; i < VE; ++i) n.v[i] += q.v[i];
     }
-    rb_store<VE>(xr + c, n);
+    row_store<VE>(xr + c, n);
 #pragma unroll
     for (int i = 0; i < VE; ++i) ss += n.v[i] * n.v[i];
     return n;
@@ -111,8 +85,8 @@ __global__ __launch_bounds__(256) void residual_branches_kernel(float* __restric
   for (int k = RB_PIECES; k < np; ++k) {
     const int c = (threadIdx.x + 256 * k) * VE;
     if (c >= D) break;
-    RbVec<VE> ta, tb;
-    if (ar != nullptr) { ta = rb_load<VE>(ar + c); tb = rb_load<VE>(br + c); }
+    RowVec<VE> ta, tb;
+    if (ar != nullptr) { ta = row_load<VE>(ar + c); tb = row_load<VE>(br + c); }
     piece(c, ta, tb);
   }
   if (h == nullptr) return;
@@ -122,10 +96,10 @@ __global__ __launch_bounds__(256) void residual_branches_kernel(float* __restric
   const float rs = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)D + eps);
   TO* hr = h + (size_t)r * ldh;
   const float g1 = hw_one ? hw[0] : 0.f;
-  auto out = [&](int c, RbVec<VE> n) {
+  auto out = [&](int c, RowVec<VE> n) {
 #pragma unroll
     for (int i = 0; i < VE; ++i) n.v[i] *= rs * (hw_one ? g1 : hw[c + i]);
-    rb_store<VE>(hr + c, n);
+    row_store<VE>(hr + c, n);
   };
 #pragma unroll
   for (int k = 0; k < RB_PIECES; ++k) {
@@ -135,7 +109,7 @@ __global__ __launch_bounds__(256) void residual_branches_kernel(float* __restric
   for (int k = RB_PIECES; k < np; ++k) {             // (a thread re-reads only what it wrote itself)
     const int c = (threadIdx.x + 256 * k) * VE;
     if (c >= D) break;
-    out(c, rb_load<VE>(xr + c));
+    out(c, row_load<VE>(xr + c));
   }
 }
 

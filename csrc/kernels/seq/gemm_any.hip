@@ -32,13 +32,14 @@ __device__ __forceinline__ void cvt_store(bf16_t* d, bf16_t v) { *d = v; }
 
 // What a kernel does with a finished accumulator element: + bias, optionally an activation (kind 1, xIELU with
 // act = {p, q}: z > 0: softplus(p) z^2 + z/2, else (1/2 + softplus(q)) (exp(z) - 1 - z) + z/2; kind 2: the square
-// of max(z, 0)), then the store as fp32 or bf16 -- so a projection whose consumer is the next matrix product writes that
+// of max(z, 0); kind 3, a decay: exp(-exp(act[column / act_n]) softplus(z))), then the store as fp32 or bf16 -- so a projection whose consumer is the next matrix product writes that
 // product's operand directly and the fp32 intermediate never reaches memory.
 struct Epi {
   const float* bias;
   const float* act;      // the activation's numbers on the device, if it has any
-  int kind;              // 0 none, 1 xIELU, 2 squared ReLU
+  int kind;              // 0 none, 1 xIELU, 2 squared ReLU, 3 decay
   int tc;                // element type of C: 0 fp32, 1 bf16
+  int act_n;             // kind 3: columns per number of act
 };
 struct EpiRegs { float ap, an; };
 __device__ __forceinline__ EpiRegs epi_regs(const Epi& e) {
@@ -46,8 +47,13 @@ __device__ __forceinline__ EpiRegs epi_regs(const Epi& e) {
   if (e.kind == 1) { r.ap = softplus_f(e.act[0]); r.an = 0.5f + softplus_f(e.act[1]); }
   return r;
 }
+// (kind 3: what a lane's column needs, before its elements are emitted)
+__device__ __forceinline__ void epi_column(const Epi& e, EpiRegs& r, int col) {
+  if (e.kind == 3) r.ap = -expf(e.act[col / e.act_n]);
+}
 __device__ __forceinline__ void emit(void* C, size_t idx, float v, const Epi& e, const EpiRegs& r) {
   if (e.kind == 2) { v = fmaxf(v, 0.f); v *= v; }
+  else if (e.kind == 3) v = expf(r.ap * softplus_f(v));
   else if (e.kind == 1) v = v > 0.f ? r.ap * v * v + 0.5f * v : r.an * (expm1f(v) - v) + 0.5f * v;
   if (e.tc == 1) reinterpret_cast<bf16_t*>(C)[idx] = f_to_bf16(v);
   else reinterpret_cast<float*>(C)[idx] = v;
@@ -91,7 +97,7 @@ __global__ __launch_bounds__(256) void gemm_nt_any(const TA* __restrict__ A, con
   __shared__ TW Ws[BN * Lds<TW>::LD];
   const int g = blockIdx.z;
   size_t cbase = 0;                      // column offset of this group in C and bias (strided batch)
-  const EpiRegs er = epi_regs(epi);
+  EpiRegs er = epi_regs(epi);
   int m0 = blockIdx.y * BM, mend = M;
   if (offs != nullptr) {
     m0 += offs[g];
@@ -136,6 +142,7 @@ __global__ __launch_bounds__(256) void gemm_nt_any(const TA* __restrict__ A, con
   const int col = n0 + wn + (lane & 31);
   if (col < N) {
     const float bv = epi.bias != nullptr ? epi.bias[cbase + col] : 0.f;
+    epi_column(epi, er, col);
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int row = m0 + wm + (r >> 2) * 8 + (lane >> 5) * 4 + (r & 3);
@@ -216,7 +223,7 @@ __global__ __launch_bounds__(64 * NWM * NWN) void gemm_nt_big(const TA* __restri
   __shared__ __attribute__((aligned(16))) TW Ws[2][TN * LD];
   const int g = blockIdx.z;
   size_t cbase = 0;
-  const EpiRegs er = epi_regs(epi);
+  EpiRegs er = epi_regs(epi);
   int m0 = blockIdx.y * TM, mend = M;
   if (offs != nullptr) {
     m0 += offs[g];
@@ -294,6 +301,7 @@ __global__ __launch_bounds__(64 * NWM * NWN) void gemm_nt_big(const TA* __restri
     const int col = n0 + wn + j * 32 + (lane & 31);
     if (col >= N) continue;
     const float bv = epi.bias != nullptr ? epi.bias[cbase + col] : 0.f;
+    epi_column(epi, er, col);
 #pragma unroll
     for (int i = 0; i < MI; ++i)
 #pragma unroll
@@ -362,7 +370,8 @@ __global__ __launch_bounds__(256) void gemm_nt_skinny(const TA* __restrict__ A, 
   for (int r = 0; r < 16; ++r) red[wave][r][lane] = acc[r];
   __syncthreads();
   if (colok) {
-    const EpiRegs er = epi_regs(epi);
+    EpiRegs er = epi_regs(epi);
+    epi_column(epi, er, col);
     const float bv = epi.bias != nullptr ? epi.bias[col] : 0.f;
 #pragma unroll
     for (int x = 0; x < 4; ++x) {
@@ -393,10 +402,11 @@ static void launch(int big, dim3 grid, hipStream_t st, const void* A, const void
 }
 
 extern "C" int fls_seq_gemm(const void* A, int ta, const void* W, int tw, void* C, int tc, const float* bias_p,
-                            const float* act, int act_kind, int M, int N, int K, int lda, int ldw, int ldc, int groups, const int* offs,
+                            const float* act, int act_kind, int act_n, int M, int N, int K, int lda, int ldw, int ldc, int groups, const int* offs,
                             long long a_gs, int a_mod, long long w_gs, long long c_gs, fls_stream_t s) {
-  if (act_kind < 0 || act_kind > 2 || (act_kind == 1 && act == nullptr)) return -1;
-  const Epi bias = {bias_p, act, act_kind, tc};
+  if (act_kind < 0 || act_kind > 3 || ((act_kind == 1 || act_kind == 3) && act == nullptr)) return -1;
+  if (act_kind == 3 && (act_n < 1 || groups != 1 || offs != nullptr)) return -1;
+  const Epi bias = {bias_p, act, act_kind, tc, act_n};
   if (M <= 0 || N <= 0) return 0;
   if (K <= 0 || groups < 1 || (ta == 1 && tw == 0)) return -1;
   const int ea = ta == 1 ? 2 : 4, ew = tw == 1 ? 2 : 4;

@@ -214,23 +214,32 @@ extern "C" int fls_seq_xielu(const float* z, int ldz, const float* act, void* y,
   return 0;
 }
 
-// y = act(gate) * up for rows [gate | up]; act: 0 = silu, 1 = gelu (tanh form)
+// y = act(gate) * up for rows [gate | up]; act: 0 = silu, 1 = gelu (tanh form), 2 = clamped: g = min(gate, limit),
+// u = clamp(up, -limit, limit), y = g sigmoid(alpha g) (u + 1)
 template <typename TO, int ACT>
-__global__ void gate_mul_kernel(const float* __restrict__ gu, int ldg, TO* __restrict__ y, int ldy, int cols) {
+__global__ __launch_bounds__(256) void gate_mul_kernel(const float* __restrict__ gu, int ldg, TO* __restrict__ y, int ldy, int cols,
+                                                       float limit, float alpha) {
   const float* gr = gu + (size_t)blockIdx.x * ldg;
   TO* yr = y + (size_t)blockIdx.x * ldy;
-  for (int c = threadIdx.x; c < cols; c += blockDim.x)
-    stf(yr, c, (ACT == 1 ? gelu_tanh_f(gr[c]) : silu_f(gr[c])) * gr[cols + c]);
+  for (int c = threadIdx.x; c < cols; c += blockDim.x) {
+    if constexpr (ACT == 2) {
+      const float g = fminf(gr[c], limit), u = fminf(fmaxf(gr[cols + c], -limit), limit);
+      stf(yr, c, g / (1.f + expf(-alpha * g)) * (u + 1.f));
+    } else {
+      stf(yr, c, (ACT == 1 ? gelu_tanh_f(gr[c]) : silu_f(gr[c])) * gr[cols + c]);
+    }
+  }
 }
 
-extern "C" int fls_seq_gate_mul(const float* gu, int ldg, void* y, int ty, int ldy, int rows, int cols, int act, fls_stream_t s) {
+extern "C" int fls_seq_gate_mul(const float* gu, int ldg, void* y, int ty, int ldy, int rows, int cols, int act, float limit,
+                                float alpha, fls_stream_t s) {
   if (rows <= 0) return 0;
-  if (act < 0 || act > 1) return -1;
+  if (act < 0 || act > 2) return -1;
   hipStream_t st = (hipStream_t)s;
-  if (ty == 1 && act == 0) hipLaunchKernelGGL((gate_mul_kernel<bf16_t, 0>), dim3(rows), dim3(256), 0, st, gu, ldg, (bf16_t*)y, ldy, cols);
-  else if (ty == 1) hipLaunchKernelGGL((gate_mul_kernel<bf16_t, 1>), dim3(rows), dim3(256), 0, st, gu, ldg, (bf16_t*)y, ldy, cols);
-  else if (act == 0) hipLaunchKernelGGL((gate_mul_kernel<float, 0>), dim3(rows), dim3(256), 0, st, gu, ldg, (float*)y, ldy, cols);
-  else hipLaunchKernelGGL((gate_mul_kernel<float, 1>), dim3(rows), dim3(256), 0, st, gu, ldg, (float*)y, ldy, cols);
+#define GATE_MUL(TO, ACT) hipLaunchKernelGGL((gate_mul_kernel<TO, ACT>), dim3(rows), dim3(256), 0, st, gu, ldg, (TO*)y, ldy, cols, limit, alpha)
+  if (ty == 1) { if (act == 0) GATE_MUL(bf16_t, 0); else if (act == 1) GATE_MUL(bf16_t, 1); else GATE_MUL(bf16_t, 2); }
+  else { if (act == 0) GATE_MUL(float, 0); else if (act == 1) GATE_MUL(float, 1); else GATE_MUL(float, 2); }
+#undef GATE_MUL
   SEQ_LAUNCH_CHECK();
   return 0;
 }
@@ -579,6 +588,148 @@ __global__ void moe_route_grouped_kernel(const float* __restrict__ logits, int l
   }
 }
 
+// Softmax scores with a correction for the choice, a wave per token: lane l holds experts l, l + 64, ...  Every choice is a
+// maximum over the wave (ties: the lower index).  FUSED (one block, few tokens): afterwards the block counts the entries
+// per expert in LDS, scans the counts and gives every entry its row, so that a decode step routes in one launch.
+#define RSG_FUSED_WAVES 16
+template <int NE, int NW, bool FUSED>
+__global__ __launch_bounds__(64 * NW) void moe_route_softmax_grouped_kernel(const float* __restrict__ logits, int ldl,
+                                                                            const float* __restrict__ corr, int T, int E, int top,
+                                                                            int groups, int keep, float scale,
+                                                                            int* __restrict__ ids, float* __restrict__ w,
+                                                                            int* __restrict__ offs, int* __restrict__ dest,
+                                                                            int* __restrict__ rows) {
+  __shared__ float choice[NW][NE * 64];
+  __shared__ int cnt[FUSED ? MOE_MAX_E : 1], start[FUSED ? MOE_MAX_E : 1];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  if constexpr (FUSED) {
+    for (int e = threadIdx.x; e < E; e += 64 * NW) cnt[e] = 0;
+    __syncthreads();
+  }
+  for (int t = blockIdx.x * NW + wave; t < T; t += gridDim.x * NW) {
+    const float* l = logits + (size_t)t * ldl;
+    float sc[NE], ch[NE];
+    float mx = -INFINITY, sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int e = lane + 64 * i;
+      sc[i] = e < E ? l[e] : -INFINITY;
+      mx = fmaxf(mx, sc[i]);
+    }
+    mx = wave_max(mx);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) { sc[i] = lane + 64 * i < E ? expf(sc[i] - mx) : 0.f; sum += sc[i]; }
+    const float inv = 1.f / wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int e = lane + 64 * i;
+      sc[i] *= inv;
+      const float c = sc[i] + (corr != nullptr && e < E ? corr[e] : 0.f);
+      ch[i] = e < E ? (c > -3e38f ? c : -3e38f) : -INFINITY;          // (an index that exists always beats one that does not)
+    }
+    if (groups > 1) {
+#pragma unroll
+      for (int i = 0; i < NE; ++i) choice[wave][lane + 64 * i] = ch[i];
+      __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+      const int per = E / groups;
+      float worth = -INFINITY;
+      if (lane < groups)
+        for (int e = 0; e < per; ++e) worth = fmaxf(worth, choice[wave][lane * per + e]);
+      bool open = lane < groups;
+      unsigned long long kept = 0ull;
+      for (int k = 0; k < keep; ++k) {
+        const float best = wave_max(open ? worth : -INFINITY);
+        const unsigned long long at = __ballot(open && worth == best);
+        const int g = __ffsll((long long)(at ? at : __ballot(open))) - 1;
+        if (lane == g) open = false;
+        kept |= 1ull << g;
+      }
+#pragma unroll
+      for (int i = 0; i < NE; ++i) {
+        const int e = lane + 64 * i;
+        if (e < E && !((kept >> (e / per)) & 1ull)) ch[i] = -INFINITY;
+      }
+      __builtin_amdgcn_wave_barrier();
+    }
+    int my_e = 0;
+    float my_s = 0.f, total = 0.f;
+    for (int k = 0; k < top; ++k) {
+      float best = -INFINITY;
+      int be = 0x7fffffff;
+#pragma unroll
+      for (int i = 0; i < NE; ++i)
+        if (ch[i] > best) { best = ch[i]; be = lane + 64 * i; }
+      const float bw = wave_max(best);
+      int e = best == bw ? be : 0x7fffffff;
+      for (int o = 32; o > 0; o >>= 1) e = min(e, __shfl_xor(e, o, 64));
+      float s = 0.f;
+#pragma unroll
+      for (int i = 0; i < NE; ++i)
+        if (lane + 64 * i == e) { s = sc[i]; ch[i] = -INFINITY; }
+      s = __shfl(s, e & 63, 64);
+      total += s;
+      if (lane == k) { my_e = e; my_s = s; }
+    }
+    if (lane < top) {
+      ids[(size_t)t * top + lane] = my_e;
+      w[(size_t)t * top + lane] = my_s * (scale / (total + 1e-20f));
+      if constexpr (FUSED) atomicAdd(&cnt[my_e], 1);
+    }
+  }
+  if constexpr (FUSED) {
+    __syncthreads();
+    if (wave == 0) {
+      const int per = (E + 63) / 64, e0 = min(E, lane * per), e1 = min(E, e0 + per);
+      int own = 0;
+      for (int e = e0; e < e1; ++e) own += cnt[e];
+      int acc = own;
+      for (int o = 1; o < 64; o <<= 1) {
+        const int v = __shfl_up(acc, o, 64);
+        if (lane >= o) acc += v;
+      }
+      if (lane == 63) offs[E] = acc;
+      acc -= own;
+      for (int e = e0; e < e1; ++e) { offs[e] = acc; start[e] = acc; acc += cnt[e]; }
+    }
+    __syncthreads();
+    // (the block's own writes of ids: visible to it after the barrier)
+    for (int i = threadIdx.x; i < T * top; i += 64 * NW) {
+      const int p = atomicAdd(&start[ids[i]], 1);
+      dest[i] = p;
+      rows[p] = i / top;
+    }
+  }
+}
+
+extern "C" int fls_seq_moe_route_softmax_grouped(const float* logits, int ldl, const float* corr, int T, int E, int top, int groups,
+                                                 int keep, float scale, int* ids, float* w, int* hist, int* offs, int* dest, int* rows,
+                                                 fls_stream_t s) {
+  if (T <= 0) return 0;
+  if (top < 1 || top > MOE_MAX_TOP || top > E || E > MOE_MAX_E || groups < 0 || groups > MOE_MAX_GROUPS) return -1;
+  if (groups > 1 && (E % groups || keep < 1 || keep > groups || keep * (E / groups) < top)) return -1;
+  hipStream_t st = (hipStream_t)s;
+  const bool fused = T <= FLS_SEQ_ROUTE_FUSED;
+#define RSG(NE)                                                                                                                     \
+  do {                                                                                                                              \
+    if (fused) hipLaunchKernelGGL((moe_route_softmax_grouped_kernel<NE, (NE > 4 ? 8 : RSG_FUSED_WAVES), true>), dim3(1),            \
+                                  dim3(64 * (NE > 4 ? 8 : RSG_FUSED_WAVES)), 0, st, logits, ldl, corr, T, E, top, groups, keep, scale, ids, w, offs, dest, rows); \
+    else hipLaunchKernelGGL((moe_route_softmax_grouped_kernel<NE, 4, false>), dim3((T + 3) / 4), dim3(256), 0, st, logits, ldl, corr, T, E, top, groups,          \
+                            keep, scale, ids, w, offs, dest, rows);                                                                 \
+  } while (0)
+  if (E <= 64) RSG(1);
+  else if (E <= 128) RSG(2);
+  else if (E <= 256) RSG(4);
+  else RSG(16);
+#undef RSG
+  SEQ_LAUNCH_CHECK();
+  if (!fused) {
+    hipLaunchKernelGGL(moe_hist_kernel, dim3((T * top + 4095) / 4096), dim3(256), 0, st, ids, T * top, E, hist);
+    SEQ_LAUNCH_CHECK();
+  }
+  return 0;
+}
+
 extern "C" int fls_seq_moe_route_grouped(const float* logits, int ldl, int T, int E, int top, int groups, int keep, float scale,
                                          int* ids, float* w, int* hist, fls_stream_t s) {
   if (T <= 0) return 0;
@@ -603,12 +754,20 @@ extern "C" int fls_seq_moe_route(const float* logits, int ldl, const float* corr
   return 0;
 }
 
-__global__ void moe_scan_kernel(const int* __restrict__ hist, int E, int* __restrict__ offs, int* __restrict__ cursor) {
-  if (threadIdx.x == 0 && blockIdx.x == 0) {
-    int acc = 0;
-    for (int e = 0; e < E; ++e) { offs[e] = acc; cursor[e] = acc; acc += hist[e]; }
-    offs[E] = acc;
+// one wave: lane l sums its run of ceil(E / 64) experts, the runs' starts come from a prefix sum over the lanes
+__global__ __launch_bounds__(64) void moe_scan_kernel(const int* __restrict__ hist, int E, int* __restrict__ offs, int* __restrict__ cursor) {
+  const int lane = threadIdx.x, per = (E + 63) / 64;
+  const int e0 = min(E, lane * per), e1 = min(E, e0 + per);
+  int own = 0;
+  for (int e = e0; e < e1; ++e) own += hist[e];
+  int acc = own;
+  for (int o = 1; o < 64; o <<= 1) {
+    const int v = __shfl_up(acc, o, 64);
+    if (lane >= o) acc += v;
   }
+  if (lane == 63) offs[E] = acc;
+  acc -= own;
+  for (int e = e0; e < e1; ++e) { offs[e] = acc; cursor[e] = acc; acc += hist[e]; }
 }
 
 extern "C" int fls_seq_moe_scan(const int* hist, int E, int* offs, int* cursor, fls_stream_t s) {
@@ -691,4 +850,4 @@ extern "C" int fls_seq_moe_combine(float* x, int ldx, const float* y, int ldy, c
   return 0;
 }
 
-extern "C" int fls_seq_version(void) { return 11; }
+extern "C" int fls_seq_version(void) { return 12; }

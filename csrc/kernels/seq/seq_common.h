@@ -34,6 +34,19 @@ __device__ __forceinline__ float block_sum_256(float v, float* red) {
   __syncthreads();
   return red[0] + red[1] + red[2] + red[3];
 }
+// v of another lane of this lane's row of 16, by a DPP control (no LDS)
+template <int CTRL>
+__device__ __forceinline__ float row_dpp(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, true));
+}
+// sum over the 16 lanes of a row; every lane gets the result (pairs, quads, then the mirrored half and the mirrored row)
+__device__ __forceinline__ float row16_sum(float v) {
+  v += row_dpp<0xB1>(v);           // lanes 1 0 3 2
+  v += row_dpp<0x4E>(v);           // lanes 2 3 0 1
+  v += row_dpp<0x141>(v);          // mirrored within 8
+  v += row_dpp<0x140>(v);          // mirrored within 16
+  return v;
+}
 __device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); }
@@ -57,8 +70,8 @@ struct AttnBlocks {
 
 // attn_paged.hip: out[t, h] from nsplit partial (maximum, sum, weighted values) records per (row, head)
 typedef void* fls_stream_t;
-// has_sink: the softmax's silent entry of score `sink` joins the total here; head_gate (nullable) [T, H]: a sigmoid gate per (row, head)
+// has_sink: the softmax's silent entry of score `sink` (sink_h given: sink_h[head]) joins the total here; head_gate (nullable) [T, H]: a sigmoid gate per (row, head)
 int seq_attn_merge(const float* part, void* out, int tc, int ldo, int T, int H, int dv, int nsplit, int gated, float out_scale,
-                   int has_sink, float sink, const float* head_gate, int ldhg, fls_stream_t s);
+                   int has_sink, float sink, const float* sink_h, const float* head_gate, int ldhg, fls_stream_t s);
 
 #define SEQ_LAUNCH_CHECK() do { hipError_t e_ = hipGetLastError(); if (e_ != hipSuccess) return (int)e_; } while (0)

@@ -7,11 +7,13 @@
 #define MAX_STREAMS 8
 
 // ------------------------------------------------------------------------------- embedding
-// out[t, c * D + j] = table[ids[t], j] * scale + pos_table[tok_pos[t], j] for every copy c
+// out[t, c * D + j] = table[ids[t], j] * scale + pos_table[tok_pos[t], j] + pair_table[pair row of (prev[t], ids[t]), j] for
+// every copy c; the pair row is a hash of the token and the one before it (prev < 0: nothing precedes, the table's last row)
 template <typename T>
 __global__ void embed_pos_kernel(const int* __restrict__ ids, const T* __restrict__ table, const T* __restrict__ pos_table,
-                                 const int* __restrict__ tok_pos, float* __restrict__ out, int D, int V, int P, float scale,
-                                 int copies) {
+                                 const int* __restrict__ tok_pos, const T* __restrict__ pair_table, const int* __restrict__ prev,
+                                 int buckets, long long mul_prev, long long mul_cur, float* __restrict__ out, int D, int V, int P,
+                                 float scale, int copies) {
   const int t = blockIdx.x;
   int id = ids[t];
   id = id < 0 ? 0 : (id >= V ? V - 1 : id);
@@ -22,22 +24,30 @@ __global__ void embed_pos_kernel(const int* __restrict__ ids, const T* __restric
     p = p < 0 ? 0 : (p >= P ? P - 1 : p);
     prow = pos_table + (size_t)p * D;
   }
+  const T* brow = nullptr;
+  if (pair_table != nullptr) {
+    const long long key = prev[t] < 0 ? buckets : ((long long)prev[t] * mul_prev + (long long)id * mul_cur) % buckets;
+    brow = pair_table + (size_t)key * D;
+  }
   float* o = out + (size_t)t * D * copies;
   for (int j = threadIdx.x; j < D; j += blockDim.x) {
     float v = ldf(row, j) * scale;
+    if (brow != nullptr) v += ldf(brow, j);
     if (prow != nullptr) v += ldf(prow, j);
     for (int c = 0; c < copies; ++c) o[(size_t)c * D + j] = v;
   }
 }
 
-extern "C" int fls_seq_embed_pos(const int* ids, const void* table, int tt, const void* pos_table, const int* tok_pos, float* out,
-                                 int T, int D, int V, int P, float scale, int copies, fls_stream_t s) {
+extern "C" int fls_seq_embed_pos(const int* ids, const void* table, int tt, const void* pos_table, const int* tok_pos,
+                                 const void* pair_table, const int* prev, int buckets, long long mul_prev, long long mul_cur,
+                                 float* out, int T, int D, int V, int P, float scale, int copies, fls_stream_t s) {
   if (T <= 0) return 0;
+  if (pair_table != nullptr && (prev == nullptr || buckets < 1 || mul_prev < 0 || mul_cur < 0)) return -1;
   if (copies < 1 || (pos_table != nullptr && (tok_pos == nullptr || P < 1))) return -1;
   if (tt == 1) hipLaunchKernelGGL((embed_pos_kernel<bf16_t>), dim3(T), dim3(256), 0, (hipStream_t)s, ids, (const bf16_t*)table,
-                                  (const bf16_t*)pos_table, tok_pos, out, D, V, P, scale, copies);
+                                  (const bf16_t*)pos_table, tok_pos, (const bf16_t*)pair_table, prev, buckets, mul_prev, mul_cur, out, D, V, P, scale, copies);
   else hipLaunchKernelGGL((embed_pos_kernel<float>), dim3(T), dim3(256), 0, (hipStream_t)s, ids, (const float*)table,
-                          (const float*)pos_table, tok_pos, out, D, V, P, scale, copies);
+                          (const float*)pos_table, tok_pos, (const float*)pair_table, prev, buckets, mul_prev, mul_cur, out, D, V, P, scale, copies);
   SEQ_LAUNCH_CHECK();
   return 0;
 }

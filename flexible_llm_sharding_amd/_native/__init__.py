@@ -130,7 +130,7 @@ def _load_kernels(path: str = _KERNELS):
     return lib
 
 
-SEQ_ABI = 11   # csrc/include/fls_seq.h
+SEQ_ABI = 12   # csrc/include/fls_seq.h
 
 
 def _load_seq():
@@ -140,7 +140,7 @@ def _load_seq():
     if lib.fls_seq_version() != SEQ_ABI:
         raise RuntimeError(f"{_SEQ} is a stale build; rebuild with python -m flexible_llm_sharding_amd._native.build")
     p, i, f, ll = c_void_p, c_int, c_float, ctypes.c_longlong
-    _bind(lib, "fls_seq_gemm", i, p, i, p, i, p, i, p, p, i, i, i, i, i, i, i, i, p, ll, i, ll, ll, p)
+    _bind(lib, "fls_seq_gemm", i, p, i, p, i, p, i, p, p, i, i, i, i, i, i, i, i, i, p, ll, i, ll, ll, p)
     _bind(lib, "fls_seq_group_rmsnorm", i, p, i, p, p, p, i, i, i, i, i, f, i, f, i, p)
     _bind(lib, "fls_seq_residual_branches", i, p, i, i, p, i, p, p, i, p, f, p, i, p, i, i, p, i, i, i, f, p)
     _bind(lib, "fls_seq_block_means", i, p, i, p, i, i, p, p, i, i, i, i, p, i, i, i, p, i, p, i, p, i, p)
@@ -153,7 +153,7 @@ def _load_seq():
     _bind(lib, "fls_seq_moe_combine", i, p, i, p, i, p, p, i, i, p, i, p, i, i, f, p)
     _bind(lib, "fls_seq_gather_rows", i, p, i, i, p, p, i, i, i, p)
     _bind(lib, "fls_seq_xielu", i, p, i, p, p, i, i, i, i, p)
-    _bind(lib, "fls_seq_gate_mul", i, p, i, p, i, i, i, i, i, p)
+    _bind(lib, "fls_seq_gate_mul", i, p, i, p, i, i, i, i, i, f, f, p)
     _bind(lib, "fls_seq_unary", i, p, i, p, i, i, i, i, i, p)
     _bind(lib, "fls_seq_head_norm_rope", i, p, i, i, i, i, i, i, p, f, p, i, p, p, p, i, i, i, i, p, i, i, i, i, f, p)
     _bind(lib, "fls_seq_delta_rule_scan", i, p, i, p, i, p, i, p, i, p, i, p, i, p, p, p, p, i, i, p, p, p, i, i, i, i, f, f, f, f, i, p, p)
@@ -161,10 +161,10 @@ def _load_seq():
     _bind(lib, "fls_seq_argmax", i, p, i, i, i, p, p)
     _bind(lib, "fls_seq_kv_store", i, p, i, p, f, p, i, p, p, i, p, i, i, i, p)
     _bind(lib, "fls_seq_attn_paged", i, p, i, i, p, i, p, i, i, p, i, i, p, p, p, i, i, i, i, i, i, f, f, p, p, i, i, i, p, f, i, i, p,
-          i, f, p, i, i, i, p, i, p, i, p, i, p)
+          i, f, p, p, i, i, i, p, i, p, i, p, i, p)
     _bind(lib, "fls_seq_attn_prefill", i, p, i, i, p, i, p, i, p, i, i, p, i, p, p, p, i, i, i, i, i, f, f, p, p, i, i, i, p, f, i,
-          i, f, p, i, i, i, p, i, p, i, p, i, p)
-    _bind(lib, "fls_seq_attn_heads", i, p, i, p, i, p, i, p, i, p, p, p, i, i, i, i, i, i, f, i, i, f, i, i, p, p)
+          i, f, p, p, i, i, i, p, i, p, i, p, i, p)
+    _bind(lib, "fls_seq_attn_heads", i, p, i, p, i, p, i, p, i, p, p, p, i, i, i, i, i, i, f, i, i, f, i, i, p, p, p, i, p)
     _bind(lib, "fls_seq_causal_conv", i, p, i, p, p, p, p, i, i, p, p, p, p, i, i, i, i, i, i, i, p)
     _bind(lib, "fls_seq_rglru_scan", i, p, i, p, i, p, p, i, p, p, i, i, p, p, p, i, i, f, p)
     _bind(lib, "fls_seq_rglru_scan_tiled", i, p, i, p, i, p, p, i, p, p, i, i, p, i, p, p, p, p, i, i, f, p)
@@ -174,7 +174,12 @@ def _load_seq():
     _bind(lib, "fls_seq_moe_place", i, p, i, i, p, p, p, p)
     _bind(lib, "fls_seq_moe_sum", i, p, i, p, p, p, i, i, i, i, p)
     _bind(lib, "fls_seq_moe_route_grouped", i, p, i, i, i, i, i, i, f, p, p, p, p)
-    _bind(lib, "fls_seq_embed_pos", i, p, p, i, p, p, p, i, i, i, i, f, i, p)
+    _bind(lib, "fls_seq_embed_pos", i, p, p, i, p, p, p, p, i, ll, ll, p, i, i, i, i, f, i, p)
+    _bind(lib, "fls_seq_moe_route_softmax_grouped", i, p, i, p, i, i, i, i, i, f, p, p, p, p, p, p, p)
+    _bind(lib, "fls_seq_rmsnorm_pair", i, p, i, p, i, p, p, i, p, p, i, i, i, i, f, p)
+    _bind(lib, "fls_seq_parallel_update", i, p, i, p, i, p, p, i, p, p, i, p, p, p, i, i, p, i, i, i, i, p)
+    _bind(lib, "fls_seq_latent_rows", i, p, i, i, i, i, p, p, f, p, i, p, p, p, i, p, i, i, i, p)
+    _bind(lib, "fls_seq_gated_delta_scan", i, p, i, p, i, p, i, p, i, p, p, p, p, i, i, p, p, p, i, i, i, i, i, i, i, f, f, f, p)
     _bind(lib, "fls_seq_streams_norm", i, p, i, p, p, p, p, i, i, i, i, i, f, p)
     _bind(lib, "fls_seq_streams_update", i, p, i, p, i, p, i, p, f, i, i, i, p, p, p, i, i, f, p)
     _bind(lib, "fls_seq_scale", i, p, i, i, i, f, p)

@@ -212,10 +212,11 @@ def _channel_delta(ctx, L, W, h, meta, name: str):
     z = ops.matmul_nt(h, W["win"])                                         # fp32 [T, q | k | v | a1 | g1 | b]
     col = lambda n: z[:, c[n][0]:c[n][0] + c[n][1]]
     qkv = ops.causal_conv(col("qkv"), W["conv"], None, st["conv"], meta, act="silu")
-    a, g = ops.matmul_nt(col("a1"), W["wa2"]), ops.matmul_nt(col("g1"), W["wg2"])
-    # unit norms, decays, step sizes, recurrence, output norm and gate
-    o = ops.gated_delta_scan(qkv, col("b"), a, g, W["dt_bias"], W["A_log"], W["mnorm"], st["state"], meta, m["heads"], m["kv_heads"],
-                             m["dim"], m["vdim"], unit_eps=UNIT_EPS, norm_eps=ctx.cfg.norm_eps, out_dtype=cdt)
+    decay = ops.matmul_nt(col("a1"), W["wa2"], bias=W["dt_bias"], decay=W["A_log"])      # the decays leave the product's epilogue
+    gate = ops.matmul_nt(col("g1"), W["wg2"])
+    # unit norms, step sizes, recurrence, output norm and gate
+    o = ops.gated_delta_scan(qkv, col("b"), decay, gate, W["mnorm"], st["state"], meta, m["heads"], m["kv_heads"], m["dim"], m["vdim"],
+                             unit_eps=UNIT_EPS, norm_eps=ctx.cfg.norm_eps, out_dtype=cdt)
     return ops.matmul_nt(o, W["wo"])
 
 

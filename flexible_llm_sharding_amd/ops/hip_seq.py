@@ -55,21 +55,30 @@ class HipSeqOps:
         self._freqs = {}
 
     # ----------------------------------------------------------------- rows
-    def embed_rows(self, ids, table, out=None, scale=1.0, pos_table=None, tok_pos=None, copies=1):
+    def embed_rows(self, ids, table, out=None, scale=1.0, pos_table=None, tok_pos=None, copies=1, bigram=None):
         T, (V, D) = ids.numel(), table.shape
         if out is None:
             out = torch.empty(T, D * copies, dtype=torch.float32, device=table.device)
         if out.dtype != torch.float32 or not out.is_contiguous() or tuple(out.shape) != (T, D * copies):
             raise TypeError("embed_rows: out must be a contiguous fp32 [T, copies * D] tensor")
         _vec(ids, "ids", T, torch.int32)
-        if pos_table is not None or copies != 1:
+        if pos_table is not None or copies != 1 or bigram is not None:
+            bt, prev, mp, mc, buckets = None, None, 0, 0, 0
+            if bigram is not None:
+                bt, prev, mp, mc = bigram
+                buckets = bt.shape[0] - 1
+                if bt.dtype != table.dtype or bt.shape[1] != D or not bt.is_contiguous() or not table.is_contiguous() or buckets < 1:
+                    raise TypeError("embed_rows: the bigram table must be laid out like table")
+                _vec(prev, "prev", T, torch.int32)
             if pos_table is not None:
                 if pos_table.dtype != table.dtype or pos_table.shape[1] != D or not pos_table.is_contiguous() or not table.is_contiguous():
                     raise TypeError("embed_rows: pos_table must be laid out like table")
                 _vec(tok_pos, "tok_pos", T, torch.int32)
             _chk(self.k.fls_seq_embed_pos(ids.data_ptr(), table.data_ptr(), _code(table, "table"),
                                           pos_table.data_ptr() if pos_table is not None else None,
-                                          tok_pos.data_ptr() if pos_table is not None else None, out.data_ptr(), T, D, V,
+                                          tok_pos.data_ptr() if pos_table is not None else None,
+                                          bt.data_ptr() if bt is not None else None, prev.data_ptr() if bt is not None else None,
+                                          buckets, int(mp), int(mc), out.data_ptr(), T, D, V,
                                           pos_table.shape[0] if pos_table is not None else 0, float(scale), int(copies), _stream()),
                  "fls_seq_embed_pos")
             return out
@@ -129,6 +138,75 @@ class HipSeqOps:
                                               ptr(wb), float(coef), ptr(add), ld(add), ptr(h), _CODE[out_dtype], D, ptr(norm_w),
                                               one, T, D, float(eps), _stream()), "fls_seq_residual_branches")
         return h
+
+    def rmsnorm_pair(self, x, w1, w2, eps, out_dtype, add=None):
+        _rows(x, "x", torch.float32)
+        T, D = x.shape
+        _vec(w1, "w1", D)
+        if w2 is not None:
+            _vec(w2, "w2", D)
+        if add is not None:
+            _rows(add, "add", torch.float32)
+            if tuple(add.shape) != (T, D):
+                raise ValueError("rmsnorm_pair: add is shaped unlike x")
+        h1 = torch.empty(T, D, dtype=out_dtype, device=x.device)
+        h2 = torch.empty(T, D, dtype=out_dtype, device=x.device) if w2 is not None else None
+        _chk(self.k.fls_seq_rmsnorm_pair(x.data_ptr(), x.stride(0), add.data_ptr() if add is not None else None,
+                                         add.stride(0) if add is not None else 0, w1.data_ptr(), h1.data_ptr(), D,
+                                         w2.data_ptr() if w2 is not None else None, h2.data_ptr() if w2 is not None else None, D,
+                                         _CODE[out_dtype], T, D, float(eps), _stream()), "fls_seq_rmsnorm_pair")
+        return h1, h2
+
+    def parallel_update_(self, x, a, wa, b=None, wb=None, moe=None):
+        _rows(x, "x", torch.float32)
+        T, D = x.shape
+        for nme, t in (("a", a), ("b", b)):
+            if t is not None:
+                _rows(t, nme, torch.float32)
+                if tuple(t.shape) != (T, D):
+                    raise ValueError(f"parallel_update_: {nme} is shaped unlike x")
+        _vec(wa, "wa", D)
+        if wb is not None:
+            _vec(wb, "wb", D)
+        if (b is not None or moe is not None) != (wb is not None) or (b is not None and moe is not None):
+            raise ValueError("parallel_update_: wb goes with b or with moe")
+        y = dest = w = ids = h = None
+        top = E = 0
+        if moe is not None:
+            y, route, h, E = moe
+            dest, w, ids = route.dest, route.w, route.ids
+            top = dest.shape[1]
+            _rows(y, "y", torch.float32)
+            _rows(h, "h")
+            if y.shape != (T * top, D) or tuple(h.shape) != (T, D) or dest.shape[0] != T:
+                raise ValueError("parallel_update_: the experts' rows do not fit")
+        ptr = lambda t: t.data_ptr() if t is not None else None
+        ld = lambda t: t.stride(0) if t is not None else 0
+        _chk(self.k.fls_seq_parallel_update(x.data_ptr(), x.stride(0), a.data_ptr(), a.stride(0), wa.data_ptr(), ptr(b), ld(b), ptr(wb),
+                                            ptr(y), ld(y), ptr(dest), ptr(w), ptr(ids), top, int(E), ptr(h),
+                                            _code(h, "h") if h is not None else 0, ld(h), T, D, _stream()), "fls_seq_parallel_update")
+        return x
+
+    def latent_rows(self, z, q_rank, r, dr, q_norm, kv_norm, eps, rot, rows, meta, out_dtype):
+        _rows(z, "z", torch.float32)
+        _rows(rows, "rows")
+        T = z.shape[0]
+        if z.shape[1] < q_rank + r + dr or rows.shape[1] < r + dr or rows.dtype != out_dtype:
+            raise ValueError("latent_rows: the rows do not fit the pool")
+        _vec(kv_norm, "kv_norm", r)
+        _vec(meta["kv_slot"], "kv_slot", T, torch.int32)
+        _vec(meta["tok_pos"], "tok_pos", T, torch.int32)
+        cq = None
+        if q_rank:
+            _vec(q_norm, "q_norm", q_rank)
+            cq = torch.empty(T, q_rank, dtype=out_dtype, device=z.device)
+        dims = int(rot[0]) if rot is not None else 0
+        freqs = self.rope_freqs(dims, rot[1], z.device) if dims else None
+        _chk(self.k.fls_seq_latent_rows(z.data_ptr(), z.stride(0), q_rank, r, dr, q_norm.data_ptr() if q_rank else None,
+                                        kv_norm.data_ptr(), float(eps), freqs.data_ptr() if dims else None, dims,
+                                        meta["tok_pos"].data_ptr(), meta["kv_slot"].data_ptr(), cq.data_ptr() if q_rank else None,
+                                        q_rank, rows.data_ptr(), rows.stride(0), _code(rows, "rows"), T, _stream()), "fls_seq_latent_rows")
+        return cq
 
     def dyt_norm(self, x, wb, alpha, out_dtype, row_idx=None):
         _rows(x, "x", torch.float32)
@@ -284,6 +362,32 @@ class HipSeqOps:
              "fls_seq_moe_place")
         return SeqRoute(ids, w, offs, rows, dest, top)
 
+    ROUTE_FUSED = 64          # FLS_SEQ_ROUTE_FUSED: up to that many tokens one launch routes, counts and places
+
+    def moe_route_softmax_grouped(self, logits, corr, top, groups, keep, scale):
+        _rows(logits, "logits", torch.float32)
+        T, E = logits.shape
+        if corr is not None:
+            _vec(corr, "corr", E)
+        dev = logits.device
+        fused = T <= self.ROUTE_FUSED
+        ids = torch.empty(T, top, dtype=torch.int32, device=dev)
+        w = torch.empty(T, top, dtype=torch.float32, device=dev)
+        ints = torch.empty(E + 1, dtype=torch.int32, device=dev) if fused else torch.zeros(3 * E + 1, dtype=torch.int32, device=dev)
+        offs, hist, cursor = ints[:E + 1], ints[E + 1:2 * E + 1], ints[2 * E + 1:]
+        dest = torch.empty(T, top, dtype=torch.int32, device=dev)
+        rows = torch.empty(T * top, dtype=torch.int32, device=dev)
+        s = _stream()
+        _chk(self.k.fls_seq_moe_route_softmax_grouped(logits.data_ptr(), logits.stride(0), corr.data_ptr() if corr is not None else None,
+                                                      T, E, top, int(groups or 0), int(keep or 0), float(scale), ids.data_ptr(),
+                                                      w.data_ptr(), hist.data_ptr(), offs.data_ptr(), dest.data_ptr(), rows.data_ptr(), s),
+             "fls_seq_moe_route_softmax_grouped")
+        if not fused:
+            _chk(self.k.fls_seq_moe_scan(hist.data_ptr(), E, offs.data_ptr(), cursor.data_ptr(), s), "fls_seq_moe_scan")
+            _chk(self.k.fls_seq_moe_place(ids.data_ptr(), T * top, top, cursor.data_ptr(), dest.data_ptr(), rows.data_ptr(), s),
+                 "fls_seq_moe_place")
+        return SeqRoute(ids, w, offs, rows, dest, top)
+
     @staticmethod
     def _block_args(blocks, kcols, vcols, page_size, dtype, B):
         """(P, kp, ldkp, vp, ldvp, table, table stride) of ``blocks`` = (block keys, block values, table, P) for a kernel."""
@@ -368,15 +472,16 @@ class HipSeqOps:
         return q_out
 
     def _gemm(self, a, w, c, bias, M, N, K, lda, ldw, ldc, groups=1, offs=None, a_gs=0, a_mod=1, w_gs=0, c_gs=0,
-              act=None, kind=0):
+              act=None, kind=0, act_n=0):
         _chk(self.k.fls_seq_gemm(a.data_ptr(), _code(a, "a"), w.data_ptr(), _code(w, "w"), c.data_ptr(), _code(c, "c"),
                                  bias.data_ptr() if bias is not None else None,
-                                 act.data_ptr() if act is not None else None, kind, M, N, K, lda, ldw, ldc, groups,
+                                 act.data_ptr() if act is not None else None, kind, act_n, M, N, K, lda, ldw, ldc, groups,
                                  offs.data_ptr() if offs is not None else None, a_gs, a_mod, w_gs, c_gs, _stream()),
              "fls_seq_gemm")
 
-    def matmul_nt(self, a, w, bias=None, xielu=None, out_dtype=torch.float32, relu2=False):
-        """a . w^T (+ bias); ``xielu`` ({p, q}) or ``relu2`` (max(z, 0)^2): that activation in the epilogue;
+    def matmul_nt(self, a, w, bias=None, xielu=None, out_dtype=torch.float32, relu2=False, decay=None):
+        """a . w^T (+ bias); ``xielu`` ({p, q}), ``relu2`` (max(z, 0)^2) or ``decay`` (rates of equal runs of columns:
+        exp(-exp(rate) softplus(z))): that activation in the epilogue;
         ``out_dtype``: the accumulator as it is (fp32) or rounded for the next product (bf16)."""
         _rows(a, "a")
         _rows(w, "w")
@@ -390,11 +495,16 @@ class HipSeqOps:
             _vec(bias, "bias", N)
         if xielu is not None:
             _vec(xielu, "xielu", 2)
-            if relu2:
-                raise ValueError("matmul_nt: one activation at a time")
+        if decay is not None and (N % decay.numel() or not decay.numel()):
+            raise ValueError("matmul_nt: decay rates do not divide the columns")
+        if (xielu is not None) + bool(relu2) + (decay is not None) > 1:
+            raise ValueError("matmul_nt: one activation at a time")
+        if decay is not None:
+            _vec(decay, "decay", decay.numel())
         c = torch.empty(M, N, dtype=out_dtype, device=a.device)
-        self._gemm(a, w, c, bias, M, N, K, a.stride(0), w.stride(0), N, act=xielu,
-                   kind=1 if xielu is not None else (2 if relu2 else 0))
+        self._gemm(a, w, c, bias, M, N, K, a.stride(0), w.stride(0), N, act=xielu if decay is None else decay,
+                   kind=1 if xielu is not None else (2 if relu2 else (3 if decay is not None else 0)),
+                   act_n=N // decay.numel() if decay is not None else 0)
         return c
 
     def block_linear(self, u, w, b, blocks, cdt):
@@ -427,16 +537,16 @@ class HipSeqOps:
                                   z.shape[0], z.shape[1], _stream()), "fls_seq_xielu")
         return y
 
-    _ACT = {"silu": 0, "gelu_tanh": 1}
+    _ACT = {"silu": 0, "gelu_tanh": 1, "clamped": 2}
     POOL_TILE_SHAPES = ((128, 128), (96, 96), (64, 64), (32, 32), (128, 64), (64, 128))    # fls_seq_attn_prefill with blocks
-    HEAD_TILE_SHAPES = ((576, 512), (320, 256), (192, 128))    # (key row, value columns) of fls_seq_attn_heads
+    HEAD_TILE_SHAPES = ((576, 512), (320, 256), (192, 128), (512, 512), (256, 256), (128, 128))    # (key row, value columns) of fls_seq_attn_heads
 
-    def gate_mul(self, gu, out_dtype, act="silu"):
+    def gate_mul(self, gu, out_dtype, act="silu", limit=0.0, alpha=1.702):
         _rows(gu, "gu", torch.float32)
         cols = gu.shape[1] // 2
         y = torch.empty(gu.shape[0], cols, dtype=out_dtype, device=gu.device)
         _chk(self.k.fls_seq_gate_mul(gu.data_ptr(), gu.stride(0), y.data_ptr(), _CODE[out_dtype], cols, gu.shape[0], cols,
-                                     self._ACT[act], _stream()), "fls_seq_gate_mul")
+                                     self._ACT[act], float(limit), float(alpha), _stream()), "fls_seq_gate_mul")
         return y
 
     def silu_mul(self, gu, out_dtype):
@@ -586,7 +696,11 @@ class HipSeqOps:
                 raise ValueError("attn_paged: head_gate is [T, H]")
         if sink is not None and gate_bias is not None:
             raise ValueError("attn_paged: a silent softmax entry and per-key sigmoid weights exclude each other")
-        extra = (1 if sink is not None else 0, float(sink or 0.0), head_gate.data_ptr() if head_gate is not None else None,
+        sink_h = sink if torch.is_tensor(sink) else None
+        if sink_h is not None:
+            _vec(sink_h, "sink", H)
+        extra = (1 if sink is not None else 0, 0.0 if sink is None or sink_h is not None else float(sink),
+                 sink_h.data_ptr() if sink_h is not None else None, head_gate.data_ptr() if head_gate is not None else None,
                  head_gate.stride(0) if head_gate is not None else 0)
         if blocks is not None and (window < 1 or chunk > 0 or keep_first or sink is not None or gate_bias is not None or r1 is not None):
             raise ValueError("attn_paged: blocks go with a plain softmax over a window")
@@ -612,18 +726,21 @@ class HipSeqOps:
             bound = min(bound, int(chunk))
         if window > 0:
             bound = min(bound, int(window) + int(keep_first) + (bound // blk[0] if blocks is not None else 0))
-        if tiles is None and q.dtype == torch.float32 and kcache.dtype == torch.bfloat16 and gate_bias is None and r1 is None \
-                and sink is None and head_gate is None and blocks is None and softcap == 0 and chunk == 0 and H // G <= 32 and Gv == G and to == 1 \
+        if q.dtype == torch.float32 and kcache.dtype == torch.bfloat16 and gate_bias is None and r1 is None \
+                and (sink is None or sink_h is not None) and blocks is None and softcap == 0 and chunk == 0 and H // G <= 32 and Gv == G and to == 1 \
                 and (d, dv) in self.HEAD_TILE_SHAPES:
-            # few rows whose heads share long key / value rows (decoding over cached latent rows): the heads of a
-            # token as the columns of one matrix-core tile, every key tile staged once for all of them
+            # rows whose heads share long key / value rows (decoding and portions over cached latent rows): the heads of
+            # a token as the columns of one matrix-core tile, every key tile staged once for all of them
             ns = max(1, min(16, 256 // max(1, T * G), bound // 32))
             part = torch.empty(T * H * ns * (dv + 4), dtype=torch.float32, device=q.device) if ns > 1 else None
             rc = self.k.fls_seq_attn_heads(q.data_ptr(), q.stride(0), kcache.data_ptr(), ldk, vcache.data_ptr(), ldv,
                                            out.data_ptr(), out.stride(0), meta["tok_seq"].data_ptr(), meta["tok_pos"].data_ptr(),
                                            table.data_ptr(), table.stride(0), T, H, G, d, dv, float(scale), int(window),
                                            int(keep_first), float(out_scale), int(page_size), ns,
-                                           part.data_ptr() if part is not None else None, _stream())
+                                           part.data_ptr() if part is not None else None,
+                                           sink_h.data_ptr() if sink_h is not None else None,
+                                           head_gate.data_ptr() if head_gate is not None else None,
+                                           head_gate.stride(0) if head_gate is not None else 0, _stream())
             if rc == 0:
                 return out
             if rc != -2:
@@ -689,6 +806,26 @@ class HipSeqOps:
                                             float(key_eps), float(norm_eps), float(out_scale), splits,
                                             raw.data_ptr() if raw is not None else None, _stream()),
              "fls_seq_delta_rule_scan")
+        return out
+
+    def gated_delta_scan(self, qkv, beta, decay, gate, norm_w, state, meta, H, G, d, dv, unit_eps, norm_eps, out_dtype):
+        T = qkv.shape[0]
+        for nme, t, n in (("qkv", qkv, 2 * G * d + H * dv), ("beta", beta, H), ("decay", decay, H * d), ("gate", gate, H * dv)):
+            _rows(t, nme, torch.float32)
+            if tuple(t.shape) != (T, n):
+                raise ValueError(f"gated_delta_scan: {nme} is {tuple(t.shape)}, not {(T, n)}")
+        _vec(norm_w, "norm_w", dv)
+        if tuple(state.shape[1:]) != (H, dv, d) or not state.is_contiguous() or state.dtype != torch.float32:
+            raise ValueError("gated_delta_scan: state must be fp32 [slots, heads, vdim, dim]")
+        out = torch.empty(T, H * dv, dtype=out_dtype, device=qkv.device)
+        one_each = meta.get("max_rows") == 1
+        raw = torch.empty(T * H * dv, dtype=torch.float32, device=qkv.device)
+        _chk(self.k.fls_seq_gated_delta_scan(qkv.data_ptr(), qkv.stride(0), beta.data_ptr(), beta.stride(0), decay.data_ptr(),
+                                             decay.stride(0), gate.data_ptr(), gate.stride(0), norm_w.data_ptr(), state.data_ptr(),
+                                             raw.data_ptr(), out.data_ptr(), _CODE[out_dtype], out.stride(0), meta["cu"].data_ptr(),
+                                             meta["pos0"].data_ptr(), meta["slot"].data_ptr(), T, meta["n_seqs"],
+                                             1 if one_each else 0, H, G, d, dv, d ** -0.5, float(unit_eps), float(norm_eps), _stream()),
+             "fls_seq_gated_delta_scan")
         return out
 
     def rglru_scan(self, u, g, lam, y, state, meta, c, out_dtype):

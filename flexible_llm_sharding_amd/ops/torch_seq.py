@@ -158,7 +158,8 @@ class TorchSeqOps:
         """o * sigmoid(g), element by element."""
         return (o.float() * torch.sigmoid(g.float())).to(out_dtype)
 
-    def matmul_nt(self, a, w, bias=None, xielu=None, out_dtype=torch.float32, relu2=False):
+    def matmul_nt(self, a, w, bias=None, xielu=None, out_dtype=torch.float32, relu2=False, decay=None):
+        """``decay`` (rates [R] of equal runs of output columns): exp(-exp(rate) softplus(y)) of the biased product."""
         if a.dtype != w.dtype:
             a = a.to(w.dtype)
         y = (a @ w.t()).float() if w.dtype == torch.float32 else (a.float() @ w.float().t())
@@ -168,6 +169,8 @@ class TorchSeqOps:
             return self.xielu(y, xielu, out_dtype)
         if relu2:
             y = torch.relu(y).square()
+        if decay is not None:
+            y = torch.exp(-torch.exp(decay.float()).repeat_interleave(y.shape[1] // decay.numel()) * F.softplus(y))
         return y.to(out_dtype)
 
     def block_linear(self, u, w, b, blocks, cdt):
@@ -485,12 +488,11 @@ class TorchSeqOps:
         out.copy_(y.to(out.dtype))
         return out
 
-    def gated_delta_scan(self, qkv, beta, a, gate, dt_bias, A_log, norm_w, state, meta, H, G, d, dv, unit_eps, norm_eps,
-                         out_dtype):
+    def gated_delta_scan(self, qkv, beta, decay, gate, norm_w, state, meta, H, G, d, dv, unit_eps, norm_eps, out_dtype):
         """Gated delta rule with a decay per head and key channel.  qkv = [q (G d) | k (G d) | v (H dv)] as convolved; head h
         reads q / k head h // (H / G).  Per head a state S carried transposed in ``state[slot]`` ([H, dv, d]):
         S <- diag(g) S,  u = sigmoid(beta) (v - S^T k),  S <- S + k u^T,  o = S^T q  with q and k divided by sqrt(sum(x^2) +
-        unit_eps), q times d^(-1/2), g = exp(-exp(A_log[h]) softplus(a + dt_bias)).  Returns
+        unit_eps), q times d^(-1/2), g = ``decay`` ([T, H d]).  Returns
         o / sqrt(mean_head(o^2) + norm_eps) * norm_w * sigmoid(gate)  (norm_w [dv], shared by the heads)."""
         T, rep = qkv.shape[0], H // G
         f = qkv.float()
@@ -499,7 +501,7 @@ class TorchSeqOps:
         k = unit(f[:, G * d:2 * G * d].reshape(T, G, d)).repeat_interleave(rep, 1)
         v = f[:, 2 * G * d:].reshape(T, H, dv)
         b = torch.sigmoid(beta.float())
-        g = torch.exp(-torch.exp(A_log.float())[None, :, None] * F.softplus(a.float() + dt_bias.float()).reshape(T, H, d))
+        g = decay.float().reshape(T, H, d)
         o = torch.empty(T, H, dv, dtype=torch.float32, device=qkv.device)
         cu, pos0, slot = meta["cu_host"], meta["pos0_host"], meta["slot"].tolist()
         for s in range(len(slot)):
