@@ -2,7 +2,8 @@
 (Kagolix beside a Mixtral-structured stack; ``--hybrid-family sisavik``: Sisavik beside Kagolix;
 ``--hybrid-family gizezen``: Gizezen beside a Kagolix stack of attention layers with experts;
 ``--hybrid-family lopilix``: Lopilix beside the Kagolix stack of attention, recurrent and state-space layers;
-``--hybrid-family nudadra``: Nudadra beside a Kagolix stack with the same mixers one after the other).
+``--hybrid-family nudadra``: Nudadra beside a Kagolix stack with the same mixers one after the other;
+``--hybrid-family numolorn``: Numolorn beside a one-stream Lopilix stack of latent attention, recurrence and experts).
 
 Random weights at sizes that resemble a real model's layers.  Three parts, one JSON line each:
 
@@ -23,7 +24,7 @@ from typing import Dict, List
 import numpy as np
 import torch
 
-from ..config import GizezenConfig, KagolixConfig, LopilixConfig, ModelConfig, NudadraConfig, SisavikConfig
+from ..config import GizezenConfig, KagolixConfig, LopilixConfig, ModelConfig, NudadraConfig, NumolornConfig, SisavikConfig
 
 PEAK_FLOPS = 2.5e15        # dense bf16 / fp16 matrix peak of one MI355X
 PEAK_BYTES = 8.0e12        # HBM3E
@@ -138,6 +139,34 @@ def kagolix_attention_mamba_config(z: dict, pairs: int = 6) -> KagolixConfig:
     att, _, mb = cfg["layers"]
     cfg["layers"] = [att, dict(mb, mlp=None)] * pairs
     return KagolixConfig.from_dict(cfg)
+
+
+def numolorn_config(z: dict, times: int = 2) -> NumolornConfig:
+    """Windowed latent attention with a dense feed-forward, latent attention with experts, a gated delta rule with experts;
+    the three layers run ``times`` times in a row on the same weights (six layer runs).  Head sizes, ranks and expert sizes of
+    the order real models use, a fifth of the router's outputs identity experts."""
+    d = z["dim"]
+    win = {"heads": z["heads"], "dim": d, "vdim": d, "kv_rank": 4 * d, "scale": d ** -0.5, "mask": {"size": z["chunk"]}}
+    lat = {"heads": z["heads"], "dim": d // 2, "rot_dim": d // 2, "vdim": d, "kv_rank": 4 * d, "q_rank": 3 * z["width"] // 4, "scale": d ** -0.5,
+           "rot": {"dims": d // 2, "base": 5.0e5}}
+    rec = {"heads": z["width"] // d, "kv_heads": z["width"] // d, "dim": d, "vdim": d, "conv": 4, "decay_rank": d, "gate_rank": d}
+    dense = {"kind": "dense", "ff": z["ff"] * 2 // 3 // 64 * 64}        # (gated: three matrices instead of two)
+    moe = {"kind": "moe", "expert": {"ff": z["eff"], "limit": 7.0},
+           "router": {"experts": z["experts"], "identity": z["experts"] // 4, "top": z["top"], "scale": 2.0, "groups": {"count": 5, "keep": 3}}}
+    layers = [{"type": "latent_attention_2", "mixer": win, "mlp": dense}, {"type": "latent_attention", "mixer": lat, "mlp": moe},
+              {"type": "channel_delta", "mixer": rec, "mlp": moe}]
+    return NumolornConfig.from_dict({"architecture": "Numolorn", "width": z["width"], "vocab": z["vocab"], "norm": {"eps": 1e-6},
+                                     "logit_scale": 0.5, "embedding": {"bigram": {"buckets": 65521, "mul_prev": 8191, "mul_cur": 31}},
+                                     "loop": {"start": 0, "stop": 3, "times": times}, "layers": layers})
+
+
+def lopilix_latent_config(z: dict, times: int = 2) -> LopilixConfig:
+    """The Lopilix stack a Numolorn stack is measured against: one residual stream, latent attention in place of both kinds
+    there, HGRN2 in place of the delta rule, the same feed-forward sizes and the same loop."""
+    cfg = lopilix_config(z, times, streams=1).to_dict()
+    att, rec, lat = cfg["layers"]
+    cfg["layers"] = [dict(lat, mlp=att["mlp"]), lat, rec]
+    return LopilixConfig.from_dict(cfg)
 
 
 def kagolix_attention_moe_config(z: dict, n_layers: int = 6) -> KagolixConfig:
@@ -848,12 +877,159 @@ def bench_nudadra_kernels(z: dict, dtype, B: int, L: int, dev) -> dict:
     return {"part": "kernels", "family": "nudadra", "dtype": str(dtype), "batch": B, "context": L, "kernels": res}
 
 
+def bench_numolorn_kernels(z: dict, dtype, B: int, L: int, dev) -> dict:
+    """The kernels of the Numolorn layers alone at the prefill shape (T = B L rows) and the decode shape (B rows at context
+    L), each beside the like kernel of an earlier family on a like shape."""
+    from ..models.numolorn import EXPERT_ALPHA, UNIT_EPS, _cols
+    from ..models.sisavik import DECAY_SCALE
+    from ..ops import get_ops
+    ops = get_ops(dev, dtype, family="hybrid")
+    es = 2 if dtype == torch.bfloat16 else 4
+    cfg = numolorn_config(z, 1)
+    win, lat, rec_ = (l.mixer for l in cfg.layers)
+    mlp = cfg.layers[1].mlp
+    D, ps = z["width"], 16
+    rt = mlp["router"]
+    E, Z, top, ff = rt["experts"], rt["experts"] + rt["identity"], rt["top"], mlp["expert"]["ff"]
+    res: Dict[str, dict] = {}
+
+    def rec(name, sec, flops=0.0, nbytes=0.0):
+        e = {"us": sec * 1e6}
+        if flops:
+            e["tflops"] = flops / sec / 1e12
+            e["of_matrix_peak"] = flops / sec / PEAK_FLOPS
+        if nbytes:
+            e["gb_s"] = nbytes / sec / 1e9
+            e["of_hbm"] = nbytes / sec / PEAK_BYTES
+        res[name] = {k: round(v, 4) for k, v in e.items()}
+
+    for tag, lens, pos0 in (("prefill", [L] * B, [0] * B), ("decode", [1] * B, [L - 1] * B)):
+        T = sum(lens)
+        meta = step_meta(B, lens, pos0, L, dev, ps)
+        meta["max_rows"] = max(lens)
+        pos = meta["pos_host"]
+        reps = 5 if tag == "prefill" else 30
+        # both latent attentions | Lopilix: latent attention without sinks, gates or a window
+        H, dl, dv, r, dr, qr = lat["heads"], lat["dim"], lat["vdim"], lat["kv_rank"], lat["rot_dim"], lat["q_rank"]
+        size = win["mask"]["size"]
+        keys = float(np.mean([p + 1 for p in pos]))
+        keys_w = float(np.mean([min(p + 1, size) for p in pos]))
+        hg, sink = torch.randn(T, H, device=dev), torch.randn(H, device=dev)
+        plain = dict(softcap=0.0, r1=None, r2=None, chunk=0, out_dtype=dtype)
+        if tag == "decode":
+            pool, pool_w = (torch.randn(meta["n_pages"], ps, n, device=dev).to(dtype) for n in (r + dr, r))
+            qa, qw = torch.randn(T, H * (r + dr), device=dev), torch.randn(T, H * r, device=dev)
+            fl, by = 2.0 * T * keys * H * (2 * r + dr), B * keys * (r + dr) * es
+            rec(f"{tag}/latent attention (folded), sinks, head gates", _timed(lambda: ops.attn_paged(
+                qa, pool, pool, meta, H, 1, r + dr, r, lat["scale"], page_size=ps, sink=sink, head_gate=hg, **plain), reps), fl, by)
+            rec(f"lopilix {tag}/latent attention (folded)", _timed(lambda: ops.attn_paged(
+                qa, pool, pool, meta, H, 1, r + dr, r, lat["scale"], page_size=ps, **plain), reps), fl, by)
+            rec(f"{tag}/windowed latent attention (folded)", _timed(lambda: ops.attn_paged(
+                qw, pool_w, pool_w, meta, H, 1, r, r, win["scale"], page_size=ps, window=size, **plain), reps),
+                4.0 * T * keys_w * H * r, B * keys_w * r * es)
+        else:
+            kf, vf = torch.randn(T, 1, H * (dl + dr), device=dev).to(dtype), torch.randn(T, 1, H * dv, device=dev).to(dtype)
+            ql = torch.randn(T, H * (dl + dr), device=dev)
+            lm = dict(meta, page_table=meta["local_table"])
+            fl = 2.0 * T * keys * H * (dl + dr + dv)
+            rec(f"{tag}/latent attention (unfolded), sinks, head gates", _timed(lambda: ops.attn_paged(
+                ql, kf, vf, lm, H, H, dl + dr, dv, lat["scale"], page_size=1, sink=sink, head_gate=hg, **plain), reps), fl)
+            al = torch.empty(T, H * dv, device=dev)
+            rec(f"lopilix {tag}/latent attention (unfolded)", _timed(lambda: ops.attn_paged(
+                ql, kf, vf, lm, H, H, dl + dr, dv, lat["scale"], page_size=1, out=al, **plain), reps), fl)
+            rec(f"{tag}/windowed latent attention (unfolded)", _timed(lambda: ops.attn_paged(
+                ql, kf, vf, lm, H, H, dl + dr, dv, win["scale"], page_size=1, window=size, **plain), reps), 2.0 * T * keys_w * H * (dl + dr + dv))
+        # norms of both latents, rotation, page write | Lopilix: latent norm and rotation into the pages, head by head
+        pool = torch.zeros(meta["n_pages"], ps, r + dr, device=dev, dtype=dtype)
+        rows = pool.view(-1, r + dr)
+        n_in = qr + r + dr + H
+        zl = torch.randn(T, n_in, device=dev)
+        qn, kn = torch.ones(qr, device=dev), torch.ones(r, device=dev)
+        rot = (dr, 5.0e5)
+        rec(f"{tag}/both latent norms, rotation, page write", _timed(lambda: ops.latent_rows(
+            zl, qr, r, dr, qn, kn, 1e-6, rot, rows, meta, dtype), reps), 0, T * (qr + r + dr) * (4 + es))
+
+        def lopilix_rows():
+            ops.head_norm_rope(zl, 1, r, qr, 0, rows, 0, 0, meta, w=kn, eps=1e-6, row_map=meta["kv_slot"])
+            ops.head_norm_rope(zl, 1, dr, qr + r, 0, rows, r, 0, meta, rot=rot, row_map=meta["kv_slot"], half=True)
+        rec(f"lopilix {tag}/latent norm, rotation, page write", _timed(lopilix_rows, reps), 0, T * (r + dr) * (4 + es))
+        # the gated delta rule | Sisavik: delta rule over heads of 64; Lopilix: HGRN2
+        Hr, d, dvr = rec_["heads"], rec_["dim"], rec_["vdim"]
+        c = _cols(cfg.layers[2])
+        zd = torch.randn(T, c["all"][1], device=dev)
+        C = c["qkv"][1]
+        cw, cst = torch.randn(C, rec_["conv"], device=dev) * 0.3, torch.zeros(B, rec_["conv"] - 1, C, device=dev)
+        rec(f"{tag}/causal convolution + silu", _timed(lambda: ops.causal_conv(zd[:, :C], cw, None, cst, meta, act="silu"), reps), 0, T * C * 8)
+        qkv = torch.randn(T, C, device=dev)
+        dec, gate, nw = torch.rand(T, Hr * d, device=dev), torch.randn(T, Hr * dvr, device=dev), torch.ones(dvr, device=dev)
+        beta = zd[:, c["b"][0]:c["b"][0] + Hr]
+        st = torch.zeros(B, Hr, dvr, d, device=dev)
+        rec(f"{tag}/gated delta scan, norm, gate", _timed(lambda: ops.gated_delta_scan(
+            qkv, beta, dec, gate, nw, st, meta, Hr, Hr, d, dvr, UNIT_EPS, 1e-6, dtype), reps), 8.0 * T * Hr * d * dvr,
+            T * Hr * (3 * d * 4 + dvr * (8 + es)) + 8.0 * B * Hr * d * dvr)
+        hd = 64
+        Hs = Hr * d // hd
+        cols = [torch.randn(T, Hs * hd, device=dev) for _ in range(6)]
+        w0, nws = torch.randn(Hs * hd, device=dev), torch.ones(Hs * hd, device=dev)
+        ss, o = torch.zeros(B, Hs, hd, hd, device=dev), torch.empty(T, Hs * hd, device=dev, dtype=dtype)
+        rec(f"sisavik {tag}/delta rule, norm, gate", _timed(lambda: ops.delta_rule_scan(
+            *cols, w0, nws, ss, meta, Hs, hd, decay_scale=DECAY_SCALE, key_eps=1e-6, norm_eps=1e-6, out_scale=1.0, out=o), reps),
+            10.0 * T * Hs * hd * hd, T * Hs * hd * (24 + es) + 8.0 * B * Hs * hd * hd)
+        lower, sh = 0.9 * torch.rand(Hr * d, device=dev), torch.zeros(B, Hr, d, dvr, device=dev)
+        rec(f"lopilix {tag}/hgrn2 scan + head norm", _timed(lambda: ops.hgrn2_scan(
+            cols[0], cols[1], cols[2], None, lower, nw, sh, meta, Hr, d, dvr, 1e-6, dtype), reps), 6.0 * T * Hr * d * dvr,
+            T * Hr * (2 * d * 4 + dvr * (12 + es)) + 8.0 * B * Hr * d * dvr)
+        ra = c["a1"][1]
+        wa = (0.02 * torch.randn(Hr * d, ra, device=dev)).to(dtype)
+        dtb, al_ = torch.randn(Hr * d, device=dev), torch.randn(Hr, device=dev)
+        a1 = zd[:, c["a1"][0]:c["a1"][0] + ra]
+        rec(f"{tag}/gemm {T}x{Hr * d}x{ra} + decay", _timed(lambda: ops.matmul_nt(a1, wa, bias=dtb, decay=al_), reps), 2.0 * T * Hr * d * ra,
+            T * (ra * 4 + Hr * d * 4) + Hr * d * ra * es)
+        rec(f"lopilix {tag}/gemm {T}x{Hr * d}x{ra}", _timed(lambda: ops.matmul_nt(a1, wa), reps), 2.0 * T * Hr * d * ra,
+            T * (ra * 4 + Hr * d * 4) + Hr * d * ra * es)
+        # the row: two norms, the update of both sublayers | one norm; a plain residual update, an expert sum
+        xs = torch.randn(T, 2 * D, device=dev)
+        x, x0 = xs[:, :D], xs[:, D:]
+        w1, w2 = torch.ones(D, device=dev), torch.ones(D, device=dev)
+        rec(f"{tag}/two norms of a row", _timed(lambda: ops.rmsnorm_pair(x, w1, w2, 1e-6, dtype), reps), 0, T * D * (4 + 2 * es))
+        rec(f"{tag}/pass entry: add, two norms", _timed(lambda: ops.rmsnorm_pair(x, w1, w2, 1e-6, dtype, add=x0), reps), 0, T * D * (12 + 2 * es))
+        rec(f"kagolix {tag}/group norm", _timed(lambda: ops.group_rmsnorm(x, w1, 1, 1e-6, dtype), reps), 0, T * D * (4 + es))
+        ya, yb = torch.randn(T, D, device=dev), torch.randn(T, D, device=dev)
+        rec(f"{tag}/update, mixer + dense", _timed(lambda: ops.parallel_update_(x, ya, w1, yb, w2), reps), 0, T * D * 16)
+        rec(f"lopilix {tag}/residual update", _timed(lambda: ops.add_scaled_(x, ya, 0.5), reps), 0, T * D * 12)
+        # routing, the experts' activation, their sum
+        logits = torch.randn(T, Z, device=dev)
+        corr = 0.1 * torch.randn(Z, device=dev)
+        g = rt["groups"]
+        rec(f"{tag}/corrected softmax routing in groups", _timed(lambda: ops.moe_route_softmax_grouped(
+            logits, corr, top, g["count"], g["keep"], 2.0), reps), 0, T * (Z * 4 + top * 20))
+        rec(f"lopilix {tag}/grouped sigmoid routing", _timed(lambda: ops.moe_route_grouped(logits, top, g["count"], g["keep"], 2.0), reps), 0,
+            T * (Z * 4 + top * 20))
+        gu = torch.randn(T * top, 2 * ff, device=dev)
+        rec(f"{tag}/clamped gate product", _timed(lambda: ops.gate_mul(gu, dtype, "clamped", limit=7.0, alpha=EXPERT_ALPHA), reps), 0, T * top * ff * (8 + es))
+        rec(f"kagolix {tag}/silu gate product", _timed(lambda: ops.gate_mul(gu, dtype, "silu"), reps), 0, T * top * ff * (8 + es))
+        route = ops.moe_route_softmax_grouped(logits, corr, top, g["count"], g["keep"], 2.0)
+        yo = torch.randn(T * top, D, device=dev)
+        h = torch.randn(T, D, device=dev).to(dtype)
+        rec(f"{tag}/update, mixer + expert sum with identities", _timed(lambda: ops.parallel_update_(x, ya, w1, wb=w2, moe=(yo, route, h, E)), reps), 0,
+            T * D * (12 + 4 * top))
+        rec(f"lopilix {tag}/expert sum", _timed(lambda: ops.moe_weighted_sum(yo, route), reps), 0, T * D * 4 * (top + 1))
+        ids, tab, bt = torch.randint(0, z["vocab"], (T,), dtype=torch.int32, device=dev), torch.randn(z["vocab"], D, device=dev).to(dtype), \
+            torch.randn(65522, D, device=dev).to(dtype)
+        rec(f"{tag}/embedding with bigrams, two copies", _timed(lambda: ops.embed_rows(ids, tab, copies=2, bigram=(bt, ids, 8191, 31)), reps), 0, T * D * (2 * es + 8))
+        rec(f"lopilix {tag}/embedding, two copies", _timed(lambda: ops.embed_rows(ids, tab, copies=2), reps), 0, T * D * (es + 8))
+        w = (0.02 * torch.randn(n_in, D, device=dev)).to(dtype)
+        rec(f"{tag}/gemm {T}x{n_in}x{D}", _timed(lambda: ops.matmul_nt(h, w), reps), 2.0 * T * n_in * D, es * (n_in * D + T * D) + 4 * T * n_in)
+    return {"part": "kernels", "family": "numolorn", "dtype": str(dtype), "batch": B, "context": L, "kernels": res}
+
+
 # family -> (its stack, the closest existing stack beside it, its kernels one by one)
 FAMILIES = {
     "lopilix": (lopilix_config, hybrid_config, bench_lopilix_kernels),
     "gizezen": (gizezen_config, kagolix_attention_moe_config, bench_gizezen_kernels),
     "sisavik": (sisavik_config, kagolix_dense_config, bench_sisavik_kernels),
     "nudadra": (nudadra_config, kagolix_attention_mamba_config, bench_nudadra_kernels),
+    "numolorn": (numolorn_config, lopilix_latent_config, bench_numolorn_kernels),
 }
 
 
@@ -869,7 +1045,7 @@ def main(a) -> int:
     if fam in FAMILIES:
         own, other, kernels = FAMILIES[fam]
         parts = {"hybrid": lambda: bench_hybrid_model(z, dtype, B, L, steps, dev, own(z), fam),
-                 "dense": lambda: bench_hybrid_model(z, dtype, B, L, steps, dev, other(z), "kagolix"),
+                 "dense": lambda: bench_hybrid_model(z, dtype, B, L, steps, dev, other(z), other(z).family),
                  "kernels": lambda: kernels(z, dtype, B, L, dev)}
     else:
         parts = {"hybrid": lambda: bench_hybrid_model(z, dtype, B, L, steps, dev),

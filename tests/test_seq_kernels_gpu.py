@@ -845,3 +845,145 @@ def test_squared_relu_in_the_epilogue(ops, cdt, tol, M, N, K):
     assert torch.equal(H.cast_rows(z, cdt), R.cast_rows(z, cdt)) and H.cast_rows(z, cdt).dtype == cdt
     z = torch.randn(M, 4 * K, device=DEV)
     assert torch.equal(H.cast_rows(z, cdt), z.to(cdt))
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+@pytest.mark.parametrize("D", [1, 36, 35, 2048, 9000])
+def test_side_by_side_rows(ops, cdt, tol, D):
+    """Two norms of a row (with and without a second weight, with a row added first) and the residual update of two
+    sublayers (plain, dense, experts with identities), on rows that are column slices of wider ones."""
+    H, R = ops
+    torch.manual_seed(D)
+    T, E, Z, top = 7, 5, 8, 3
+    wide = torch.randn(T, 2 * D, device=DEV)
+    w1, w2 = torch.randn(D, device=DEV), torch.randn(D, device=DEV)
+    for add in (False, True):
+        for second in (w2, None):
+            xa, xb = wide.clone(), wide.clone()
+            a1, a2 = H.rmsnorm_pair(xa[:, :D], w1, second, 1e-5, cdt, add=xa[:, D:] if add else None)
+            b1, b2 = R.rmsnorm_pair(xb[:, :D], w1, second, 1e-5, cdt, add=xb[:, D:] if add else None)
+            close(a1, b1, tol)
+            close(xa, xb, 1e-6)
+            assert (a2 is None) == (b2 is None)
+            if a2 is not None:
+                close(a2, b2, tol)
+    a, b = torch.randn(T, D, device=DEV), torch.randn(T, D, device=DEV)
+    h, y = torch.randn(T, D, device=DEV).to(cdt), torch.randn(T * top, D, device=DEV)
+    route = R.moe_route_softmax_grouped(torch.randn(T, Z, device=DEV) * 2, None, top, 4, 3, 1.3)
+    assert bool((route.ids >= E).any()) and bool((route.ids < E).any())
+    y[int(route.offs[E]):] = float("nan")                                   # (rows of identity experts are never made)
+    for kw in ({}, {"b": b, "wb": w2}, {"wb": w2, "moe": (y, route, h, E)}):
+        xa, xb = wide.clone(), wide.clone()
+        H.parallel_update_(xa[:, :D], a, w1, **kw)
+        kr = dict(kw, moe=(y.nan_to_num(), route, h, E)) if "moe" in kw else kw
+        R.parallel_update_(xb[:, :D], a, w1, **kr)
+        close(xa, xb, 1e-5)
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+@pytest.mark.parametrize("qr,r,dr,rot", [(9, 11, 8, 8), (1536, 512, 64, 64), (0, 40, 0, 0), (4, 12, 3, 2), (300, 1, 0, 0), (0, 512, 512, 64)])
+def test_latent_rows(ops, cdt, tol, qr, r, dr, rot):
+    """Both latents' norms, the rotated key part and the place in the pool, in one pass; other rows of the pool stay."""
+    H, R = ops
+    torch.manual_seed(qr + r)
+    md, n_pages, _ = meta_of([5, 40, 1], [0, 7, 3000], DEV)
+    T = 46
+    z = torch.randn(T, qr + r + dr + 3, device=DEV)
+    qn, kn = torch.randn(max(qr, 1), device=DEV), torch.randn(r, device=DEV)
+    pa = torch.randn(n_pages * 16, r + dr, device=DEV).to(cdt)
+    pb = pa.clone()
+    args = (z, qr, r, dr, qn if qr else None, kn, 1e-5, (rot, 500.0) if rot else None)
+    a, b = H.latent_rows(*args, pa, md, cdt), R.latent_rows(*args, pb, md, cdt)
+    close(pa, pb, tol)
+    assert (a is None) == (qr == 0)
+    if qr:
+        close(a, b, tol)
+
+
+@pytest.mark.parametrize("heads,kv,d,dv", [(4, 2, 7, 9), (3, 3, 1, 1), (2, 1, 64, 64), (3, 3, 48, 130), (2, 2, 128, 128), (6, 2, 130, 20),
+                                           (1, 1, 256, 300), (2, 1, 100, 512), (2, 2, 256, 128), (16, 8, 64, 64)])
+def test_gated_delta_scan_carries_state(ops, heads, kv, d, dv):
+    """The gated delta rule over unequal requests, some continuing from states in scattered slots: portions longer and shorter
+    than a staged round, one row each (the fused form), strong and weak decays; outputs and states."""
+    H, R = ops
+    torch.manual_seed(heads + d)
+    for lens, pos0 in (([33, 1, 7, 16], [0, 5, 12, 3]), ([1, 1, 1], [4, 0, 9]), ([50], [0]), ([2, 2], [0, 40])):
+        md, _, n_slots = meta_of(lens, pos0, DEV)
+        T = sum(lens)
+        qkv = torch.randn(T, 2 * kv * d + heads * dv, device=DEV)
+        zz = torch.randn(T, heads + 3, device=DEV)
+        dec = torch.rand(T, heads * d, device=DEV) ** 3
+        dec[:, ::5] = 1.0
+        dec[:, 1::7] = 0.0
+        gate, nw = torch.randn(T, heads * dv, device=DEV), 1 + 0.2 * torch.randn(dv, device=DEV)
+        st = torch.randn(n_slots, heads, dv, d, device=DEV)
+        for cdt, tol in ((torch.float32, 2e-4), (torch.bfloat16, 2e-2)):
+            s1, s2 = st.clone(), st.clone()
+            a = H.gated_delta_scan(qkv, zz[:, 2:2 + heads], dec, gate, nw, s1, md, heads, kv, d, dv, 1e-6, 1e-5, cdt)
+            b = R.gated_delta_scan(qkv, zz[:, 2:2 + heads], dec, gate, nw, s2, md, heads, kv, d, dv, 1e-6, 1e-5, cdt)
+            close(a, b, tol)
+            close(s1, s2, 2e-4)                                             # (slots of nobody in the step stay as they were)
+
+
+@pytest.mark.parametrize("T,E,top,groups,keep", [(50, 8, 2, 4, 3), (7, 12, 3, 4, 2), (300, 5, 2, 5, 3), (33, 6, 6, 2, 2), (20, 7, 1, 0, 0),
+                                                 (64, 64, 8, 8, 4), (65, 64, 8, 8, 4), (9, 128, 16, 64, 9), (70, 150, 8, 10, 4), (3, 1024, 16, 32, 5),
+                                                 (1, 3, 2, 3, 2), (500, 1024, 4, 0, 0)])
+def test_corrected_softmax_routing_in_groups(ops, T, E, top, groups, keep):
+    """Few tokens (one launch routes, counts and places) and many; corrections that make every choice score negative, none."""
+    H, R = ops
+    torch.manual_seed(T + E)
+    logits = torch.randn(T, E + 3, device=DEV)[:, 1:1 + E] * 2
+    for corr in (0.3 * torch.randn(E, device=DEV), 0.3 * torch.randn(E, device=DEV) - 3.0, None):
+        a, b = (o.moe_route_softmax_grouped(logits, corr, top, groups, keep, 1.9) for o in (H, R))
+        assert torch.equal(a.ids.cpu(), b.ids.cpu())
+        close(a.w, b.w, 1e-5)
+        assert torch.equal(a.offs.cpu(), b.offs.cpu())
+        offs, dest = a.offs.cpu().long(), a.dest.cpu().long()
+        assert bool(((dest >= offs[a.ids.cpu().long()]) & (dest < offs[a.ids.cpu().long() + 1])).all())
+        assert torch.equal(a.rows.cpu().long()[dest], torch.arange(T)[:, None].expand(T, top))
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+def test_clamped_gates_decays_and_bigram_rows(ops, cdt, tol):
+    """The clamped gate product; a product whose epilogue turns it into decays (64- and 128-row tiles, few rows, an odd K);
+    embedding rows with hashed bigrams (large multipliers, first tokens), one and two copies."""
+    H, R = ops
+    torch.manual_seed(3)
+    gu = torch.randn(9, 2 * 300, device=DEV) * 4
+    gu[0, :4] = torch.tensor([90.0, -90.0, 1.5, -1.5], device=DEV)
+    for limit in (1.5, 1e4):
+        close(H.gate_mul(gu, cdt, "clamped", limit=limit, alpha=1.702), R.gate_mul(gu, cdt, "clamped", limit=limit, alpha=1.702), tol)
+    for M, N, K, n in ((5, 60, 33, 6), (3, 96, 64, 3), (150, 256, 24, 2), (70, 40, 16, 40)):
+        a, w = torch.randn(M, K, device=DEV), (0.3 * torch.randn(N, K, device=DEV)).to(cdt)
+        b, rates = torch.randn(N, device=DEV), torch.randn(n, device=DEV)
+        close(H.matmul_nt(a, w, bias=b, decay=rates), R.matmul_nt(a, w, bias=b, decay=rates), tol)
+    V, D, n = 40, 50, 23
+    ids = torch.randint(0, V, (12,), dtype=torch.int32, device=DEV)
+    prev = torch.randint(-1, V, (12,), dtype=torch.int32, device=DEV)
+    prev[3] = -1
+    tab, bt = torch.randn(V, D, device=DEV).to(cdt), torch.randn(n + 1, D, device=DEV).to(cdt)
+    for mp, mc in ((7, 3), (1 << 30, (1 << 30) + 1), (0, 1)):
+        for copies in (1, 2):
+            close(H.embed_rows(ids, tab, copies=copies, bigram=(bt, prev, mp, mc)), R.embed_rows(ids, tab, copies=copies, bigram=(bt, prev, mp, mc)), 1e-6)
+
+
+@pytest.mark.parametrize("cdt,tol", DTYPES)
+@pytest.mark.parametrize("Hh,G,d,dv", [(3, 3, 14, 5), (4, 4, 128, 128), (6, 1, 64, 64), (5, 1, 576, 512), (32, 1, 512, 512), (7, 1, 256, 256), (3, 1, 128, 128),
+                                       (40, 1, 128, 128)])
+def test_attention_with_a_sink_per_head(ops, cdt, tol, Hh, G, d, dv):
+    """A silent softmax entry of its own score in every head, loud and next to nothing, with head gates and windows, through
+    every attention kernel: prompts, single rows over short contexts, single rows whose keys are cut into ranges, portions."""
+    H, R = ops
+    torch.manual_seed(Hh + d)
+    sink = torch.randn(Hh, device=DEV) * 3
+    sink[0] = -60.0
+    for lens, pos0 in (([40, 150], [0, 33]), ([1, 1, 1], [0, 20, 900]), ([1], [1500]), ([2, 3], [500, 0])):
+        md, n_pages, _ = meta_of(lens, pos0, DEV)
+        kc = (torch.randn(n_pages, 16, G * d, device=DEV) * 0.3).to(cdt)
+        vc = kc if G == 1 and dv <= d else (torch.randn(n_pages, 16, G * dv, device=DEV) * 0.3).to(cdt)
+        q = torch.randn(sum(lens), Hh * d, device=DEV)
+        hg = torch.randn(sum(lens), Hh + 2, device=DEV)[:, 1:1 + Hh]
+        for window in (0, 50):
+            for s, g in ((sink, hg), (sink, None), (None, hg)):
+                kw = dict(scale=d ** -0.5, softcap=0.0, r1=None, r2=None, chunk=0, page_size=16, out_dtype=cdt, window=window, sink=s, head_gate=g)
+                close(H.attn_paged(q, kc, vc, md, Hh, G, d, dv, **kw), R.attn_paged(q, kc, vc, md, Hh, G, d, dv, **kw), tol)
