@@ -126,7 +126,7 @@ __global__ __launch_bounds__(64 * WAVES) void gated_delta_kernel(const float* __
     }
     __syncthreads();
     load(t0 + TT);
-#pragma unroll 2
+#pragma unroll 1
     for (int j = 0; j < rows; ++j) {                 // (no barrier in here: a lane's columns are its own)
       float p1[CN], p2[CN];
       float kf[RPL];
@@ -247,9 +247,9 @@ extern "C" int fls_seq_gated_delta_scan(const float* qkv, int ldq, const float* 
     }
   }
   if (raw == nullptr) return -1;
-  // as many columns a lane as still leave the chip a wave per SIMD: the factors read from LDS serve them all
+  // as many columns a lane as still leave the chip two waves per SIMD: the factors read from LDS serve them all
   int cn = rpl == 16 ? 2 : 4;
-  while (cn > 1 && (long long)H * B * ((dv + 16 * cn - 1) / (16 * cn)) * 4 < 1024) cn /= 2;
+  while (cn > 1 && (long long)H * B * ((dv + 16 * cn - 1) / (16 * cn)) * 4 < 2048) cn /= 2;
 #define GD_P(R, C) hipLaunchKernelGGL((gated_delta_kernel<R, C, 4, 16, false, float>), dim3((dv + 16 * C - 1) / (16 * C), H, B), dim3(256), 0, st, \
                                       GD_ARGS, raw, H * dv, GD_TAIL)
   if (rpl == 4) { if (cn == 1) GD_P(4, 1); else if (cn == 2) GD_P(4, 2); else GD_P(4, 4); }

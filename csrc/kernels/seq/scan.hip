@@ -56,6 +56,30 @@ __global__ void causal_conv_rows_kernel(const float* __restrict__ x, int ldx, co
     xv[j] = 0.f;
   }
   const float bias = b != nullptr ? b[c] : 0.f;
+  if (t1 - t0 == CONV_ROWS && !fuse_state && tok_seq[t0] == tok_seq[t1 - 1]) {
+    // a full run inside one request: all its loads are issued at once, the sums follow from registers
+    const int s = tok_seq[t0], tl = t0 - cu[s];
+    const bool carried = pos0[s] > 0;
+    const float* hist = state + (size_t)slot[s] * (taps - 1) * C;
+    float xr[CONV_ROWS];
+#pragma unroll
+    for (int r = 0; r < CONV_ROWS; ++r) xr[r] = x[(size_t)(t0 + r) * ldx + c];
+#pragma unroll
+    for (int j = 1; j < CONV_MAX_TAPS; ++j)
+      if (j < taps) {
+        if (tl - j >= 0) xv[j] = x[(size_t)(t0 - j) * ldx + c];
+        else if (carried) xv[j] = hist[(size_t)(taps - 1 + tl - j) * C + c];
+      }
+#pragma unroll
+    for (int r = 0; r < CONV_ROWS; ++r) {
+      float acc = bias;
+#pragma unroll
+      for (int j = 0; j < CONV_MAX_TAPS; ++j) acc += wv[j] * (r >= j ? xr[r >= j ? r - j : 0] : xv[r >= j ? 0 : j - r]);
+      if (residual) acc += xr[r];
+      stf(out + (size_t)(t0 + r) * ldo, c, act == 1 ? silu_f(acc) : acc);
+    }
+    return;
+  }
   int prev = -1;
   for (int t = t0; t < t1; ++t) {
     const int s = tok_seq[t];
