@@ -362,7 +362,7 @@ class HipSeqOps:
              "fls_seq_moe_place")
         return SeqRoute(ids, w, offs, rows, dest, top)
 
-    ROUTE_FUSED = 64          # FLS_SEQ_ROUTE_FUSED: up to that many tokens one launch routes, counts and places
+    ROUTE_FUSED = 64          # (the limit in csrc/include/fls_seq.h) up to that many tokens one launch routes, counts and places
 
     def moe_route_softmax_grouped(self, logits, corr, top, groups, keep, scale):
         _rows(logits, "logits", torch.float32)
